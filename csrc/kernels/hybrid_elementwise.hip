@@ -8,7 +8,7 @@
 //
 //  * embedding_f32      x[t] = table[ids[t]] * scale (+ pos_table[positions[t]]) as fp32 (two
 //                       copies: the stream and the loop input)
-//  * resadd_groupnorm   x = keep * x + mult * y + bias; h = grouped RMS norm of x * gain (S out,
+//  * resadd_groupnorm   x = keep * x + mult * y + bias + add; h = grouped RMS norm of x * gain (S out,
 //                       or unrounded fp32 for a consumer that mixes rows first)
 //  * token_shift        u[t] = h[t] + (h[t-1] - h[t]) * mu over the normed fp32 rows, h[t-1] of a
 //                       portion's first row from the sequence's state slot
@@ -53,15 +53,15 @@ __global__ void __launch_bounds__(256) embedding_f32_kernel(
   if (x0 != nullptr) x0[gid] = v;
 }
 
-// One workgroup per row. x (fp32, in place): x = keep * x + mult * y + bias, y and bias may be
-// null. The row is cut into `groups` equal parts, each scaled by its own rsqrt(mean(sq) + eps);
+// One workgroup per row. x (fp32, in place): x = keep * x + mult * y + bias + add, y, bias and
+// the rows `add` (fp32, x's layout) may be null. The row is cut into `groups` equal parts, each scaled by its own rsqrt(mean(sq) + eps);
 // h = that * w. h may be null (the last layer's add). rows_idx (nullable) selects source rows
 // (the final norm of the rows whose logits are wanted); it excludes y / bias / the write-back.
 template <typename S>
 __global__ void __launch_bounds__(256) resadd_groupnorm_kernel(
     float* __restrict__ x, const float* __restrict__ y, int ldy, const S* __restrict__ bias,
-    float keep, float mult, const S* __restrict__ w, void* __restrict__ h, int ldh, int dim,
-    int groups, float eps, const long* __restrict__ rows_idx, bool vec4, float gain,
+    const float* __restrict__ add, float keep, float mult, const S* __restrict__ w,
+    void* __restrict__ h, int ldh, int dim, int groups, float eps, const long* __restrict__ rows_idx, bool vec4, float gain,
     bool h_f32, float w_offset) {
   extern __shared__ __attribute__((aligned(16))) float row[];   // dim floats + group scales
   float* gsum = row + dim;
@@ -69,7 +69,7 @@ __global__ void __launch_bounds__(256) resadd_groupnorm_kernel(
   const long src = rows_idx ? rows_idx[r] : r;
   float* xr = x + src * dim;
   for (int g = threadIdx.x; g < groups; g += blockDim.x) gsum[g] = 0.f;
-  const bool update = rows_idx == nullptr && (y != nullptr || bias != nullptr || keep != 1.f);
+  const bool update = rows_idx == nullptr && (y != nullptr || bias != nullptr || add != nullptr || keep != 1.f);
   if (vec4) {                               // 16-byte loads and stores of the fp32 rows
     for (int c = threadIdx.x * 4; c < dim; c += blockDim.x * 4) {
       f32x4 v = *reinterpret_cast<const f32x4*>(xr + c);
@@ -81,6 +81,7 @@ __global__ void __launch_bounds__(256) resadd_groupnorm_kernel(
 #pragma unroll
           for (int u = 0; u < 4; ++u) v[u] += ldf(bias + c + u);
         }
+        if (add != nullptr) v += *reinterpret_cast<const f32x4*>(add + (long)r * dim + c);
         if (update) *reinterpret_cast<f32x4*>(xr + c) = v;
       }
       *reinterpret_cast<f32x4*>(row + c) = v;
@@ -92,6 +93,7 @@ __global__ void __launch_bounds__(256) resadd_groupnorm_kernel(
         v = keep != 0.f ? v * keep : 0.f;
         if (y != nullptr) v += mult * y[(long)r * ldy + c];
         if (bias != nullptr) v += ldf(bias + c);
+        if (add != nullptr) v += add[(long)r * dim + c];
         if (update) xr[c] = v;
       }
       row[c] = v;
@@ -424,8 +426,8 @@ extern "C" int dli_embedding_f32(float* x, float* x0, const int* ids, const void
 }
 
 extern "C" int dli_resadd_groupnorm(float* x, const float* y, int ldy, const void* bias,
-                                    float keep, float mult, const void* w, void* h, int ldh,
-                                    int rows, int dim, int groups, float eps,
+                                    const float* add, float keep, float mult, const void* w,
+                                    void* h, int ldh, int rows, int dim, int groups, float eps,
                                     const long* rows_idx, float gain, int h_f32, float w_offset,
                                     int dt, hipStream_t st) {
   if (rows <= 0) return 0;
@@ -433,13 +435,14 @@ extern "C" int dli_resadd_groupnorm(float* x, const float* y, int ldy, const voi
     return (int)hipErrorInvalidValue;
   const size_t sh = (size_t)(dim + groups) * 4;
   const bool vec4 = dim % 4 == 0 && (uintptr_t)x % 16 == 0 &&
-                    (y == nullptr || ((uintptr_t)y % 16 == 0 && ldy % 4 == 0));
+                    (y == nullptr || ((uintptr_t)y % 16 == 0 && ldy % 4 == 0)) &&
+                    (uintptr_t)add % 16 == 0;
   DT_SWITCH(dt,
             (resadd_groupnorm_kernel<u16><<<rows, 256, sh, st>>>(
-                x, y, ldy, (const u16*)bias, keep, mult, (const u16*)w, h, ldh, dim, groups,
+                x, y, ldy, (const u16*)bias, add, keep, mult, (const u16*)w, h, ldh, dim, groups,
                 eps, rows_idx, vec4, gain, h_f32 != 0, w_offset)),
             (resadd_groupnorm_kernel<float><<<rows, 256, sh, st>>>(
-                x, y, ldy, (const float*)bias, keep, mult, (const float*)w, h, ldh, dim,
+                x, y, ldy, (const float*)bias, add, keep, mult, (const float*)w, h, ldh, dim,
                 groups, eps, rows_idx, vec4, gain, h_f32 != 0, w_offset)));
   DLI_RETURN_LAUNCH();
 }

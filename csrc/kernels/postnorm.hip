@@ -12,7 +12,8 @@
 //  * add_rmsnormed     x += y / sqrt(mean(y^2) + eps) * w in place, and the S copy of x
 //  * side_gate         gelu_tanh(gate) * table[id, col0 + c] -> S (a per-layer slice of a
 //                      second embedding table gates a small projection)
-//  * rmsnorm_cols      RMS norm * w (* sigmoid(gate)) of a column slice of an fp32 projection -> S
+//  * rmsnorm_cols      RMS norm (* w) (* sigmoid(gate), or silu(gate)) of a column slice of an fp32
+//                      projection -> S
 //  * latent_prepare    latent attention with the queries and the compressed kv in separate
 //                      projections: RMS norm of the latent -> cache, rotary on the shared key ->
 //                      cache (skipped by a layer that reads another layer's cache), rotary on
@@ -202,18 +203,23 @@ __global__ void __launch_bounds__(256) side_gate_kernel(
 }
 
 // One wave per row.
+// sigmoid(g), or silu(g)
+__device__ __forceinline__ float gate_of(float g, bool silu) {
+  return (silu ? g : 1.f) / (1.f + expf(-g));
+}
+
 template <typename S>
 __global__ void __launch_bounds__(256) rmsnorm_cols_kernel(
     S* __restrict__ out, const float* __restrict__ src, int lds, const S* __restrict__ w, int T,
     int n, float eps, bool vec4, const float* __restrict__ gate, int ldg, int groups, int ldo,
-    float out_scale) {
+    float out_scale, bool silu) {
   // a row = one of `groups` parts (n wide each, normed by itself) of a token's row
   const int lane = threadIdx.x & 63;
   const int row = blockIdx.x * (blockDim.x >> 6) + (threadIdx.x >> 6);
   if (row >= T * groups) return;
   const int t = row / groups, go = (row % groups) * n;
   const float* r = src + (long)t * lds + go;
-  w += go;
+  if (w != nullptr) w += go;
   out += (long)t * ldo + go;
   if (gate != nullptr) gate += (long)t * ldg + go;
   float s = 0.f;
@@ -225,11 +231,12 @@ __global__ void __launch_bounds__(256) rmsnorm_cols_kernel(
     s = wave_sum(s);
     const float rs = 1.f / sqrtf(s / (float)n + eps);
     for (int c = lane * 4; c < n; c += 256) {
-      f32x4 v = *reinterpret_cast<const f32x4*>(r + c) * rs * ld4(w + c);
+      f32x4 v = *reinterpret_cast<const f32x4*>(r + c) * rs;
+      if (w != nullptr) v *= ld4(w + c);
       if (gate != nullptr) {
         const f32x4 g = *reinterpret_cast<const f32x4*>(gate + c);
 #pragma unroll
-        for (int u = 0; u < 4; ++u) v[u] *= 1.f / (1.f + expf(-g[u]));
+        for (int u = 0; u < 4; ++u) v[u] *= gate_of(g[u], silu);
       }
       st4(out + c, v * out_scale);
     }
@@ -239,8 +246,9 @@ __global__ void __launch_bounds__(256) rmsnorm_cols_kernel(
   s = wave_sum(s);
   const float rs = 1.f / sqrtf(s / (float)n + eps);
   for (int c = lane; c < n; c += 64) {
-    float v = r[c] * rs * ldf(w + c);
-    if (gate != nullptr) v *= 1.f / (1.f + expf(-gate[c]));
+    float v = r[c] * rs;
+    if (w != nullptr) v *= ldf(w + c);
+    if (gate != nullptr) v *= gate_of(gate[c], silu);
     stf(out + c, v * out_scale);
   }
 }
@@ -249,7 +257,8 @@ __global__ void __launch_bounds__(256) rmsnorm_cols_kernel(
 template <typename S>
 __global__ void __launch_bounds__(256) rmsnorm_cols_block_kernel(
     S* __restrict__ out, const float* __restrict__ src, int lds, const S* __restrict__ w, int n,
-    float eps, const float* __restrict__ gate, int ldg, int groups, int ldo, float out_scale) {
+    float eps, const float* __restrict__ gate, int ldg, int groups, int ldo, float out_scale,
+    bool silu) {
   __shared__ float red[16];
   const int t = blockIdx.x / groups, go = (blockIdx.x % groups) * n;
   const float* r = src + (long)t * lds + go;
@@ -258,8 +267,9 @@ __global__ void __launch_bounds__(256) rmsnorm_cols_block_kernel(
   s = block_sum(s, red);
   const float rs = 1.f / sqrtf(s / (float)n + eps);
   for (int c = threadIdx.x; c < n; c += blockDim.x) {
-    float v = r[c] * rs * ldf(w + go + c);
-    if (gate != nullptr) v *= 1.f / (1.f + expf(-gate[(long)t * ldg + go + c]));
+    float v = r[c] * rs;
+    if (w != nullptr) v *= ldf(w + go + c);
+    if (gate != nullptr) v *= gate_of(gate[(long)t * ldg + go + c], silu);
     stf(out + (long)t * ldo + go + c, v * out_scale);
   }
 }
@@ -498,16 +508,17 @@ extern "C" int dli_side_gate(void* out, const float* gate, int ldg, const int* i
 
 extern "C" int dli_rmsnorm_cols(void* out, const float* src, int lds, const void* w, int T, int n,
                                 float eps, const float* gate, int ldg, int groups, int ldo,
-                                float out_scale, int dt, hipStream_t st) {
+                                float out_scale, int silu, int dt, hipStream_t st) {
   if (T <= 0) return 0;
   if (n < 1 || groups < 1) return (int)hipErrorInvalidValue;
   if ((long)T * groups <= 512 && n >= 1024) {
     DT_SWITCH(dt,
               (rmsnorm_cols_block_kernel<u16><<<T * groups, 256, 0, st>>>(
-                  (u16*)out, src, lds, (const u16*)w, n, eps, gate, ldg, groups, ldo, out_scale)),
+                  (u16*)out, src, lds, (const u16*)w, n, eps, gate, ldg, groups, ldo, out_scale,
+                  silu != 0)),
               (rmsnorm_cols_block_kernel<float><<<T * groups, 256, 0, st>>>(
                   (float*)out, src, lds, (const float*)w, n, eps, gate, ldg, groups, ldo,
-                  out_scale)));
+                  out_scale, silu != 0)));
     DLI_RETURN_LAUNCH();
   }
   const int nb = (int)(((long)T * groups + 3) / 4);
@@ -516,10 +527,11 @@ extern "C" int dli_rmsnorm_cols(void* out, const float* src, int lds, const void
   DT_SWITCH(dt,
             (rmsnorm_cols_kernel<u16><<<nb, 256, 0, st>>>((u16*)out, src, lds, (const u16*)w, T,
                                                           n, eps, vec4, gate, ldg, groups, ldo,
-                                                          out_scale)),
+                                                          out_scale, silu != 0)),
             (rmsnorm_cols_kernel<float><<<nb, 256, 0, st>>>((float*)out, src, lds,
                                                             (const float*)w, T, n, eps, vec4,
-                                                            gate, ldg, groups, ldo, out_scale)));
+                                                            gate, ldg, groups, ldo, out_scale,
+                                                            silu != 0)));
   DLI_RETURN_LAUNCH();
 }
 

@@ -15,9 +15,13 @@
 //     n_t . q_t = A_t (n_0 . q_t) + sum_{j <= t} b_j (prod_{j < i <= t} a_i) (k_j . q_t),
 //   A_t = prod_{i <= t} a_i, so the chunk's key-query products and the carried vector n_0 (LDS,
 //   updated once a chunk) give every token's normaliser in parallel, beside the walk.
+// FORM 2, retention: as FORM 0 without activations; the first `rot` dims of q and k rotate
+//   (dimension i with i + rot/2, by the step's table of cosines | sines), k times d^(-1/2); o_t
+//   is divided by its RMS per head and multiplied by silu(gate_t) -> S. Portions of more than
+//   a few tokens run the chunk form of retention.hip instead.
 //
 // Projection row of a token (fp32): [H*d q | H*d k | H*dv v | H*dv gate | H zi | H zf] (FORM 0
-// reads q, k, v only). State: [slots, H, d, dv]; FORM 1 also nstate [slots, H, d + 1] = n, then
+// reads q, k, v only, FORM 2 also the gate). State: [slots, H, d, dv]; FORM 1 also nstate [slots, H, d + 1] = n, then
 // m. A step's tokens of one sequence are consecutive rows [cu[s], cu[s+1]);
 // positions[cu[s]] == 0 starts from a zero state whatever the slot held; sequences with slot
 // < 0 (padding rows of a captured decode step) get zeros.
@@ -28,7 +32,7 @@
 // keeps the state in LDS. Tokens are taken in chunks of TC: activations and gates of the
 // chunk in parallel (the running maximum by one wave), the walk without barriers, the
 // chunk's read-outs finished one wave per token. With several column blocks a head's RMS norm
-// cannot happen here: FORM 1 then leaves o_t in fp32 (`raw`) for a norm kernel.
+// cannot happen here: FORMs 1 and 2 then leave o_t in fp32 (`raw`) for a norm kernel.
 #include "common.h"
 
 namespace {
@@ -58,8 +62,10 @@ struct ScalarRecArgs {
   float* state; float* nstate;
   const int* slots; const int* cu; const int* positions;
   void* out; int ldo; float out_scale;
-  float* raw;                     // FORM 1, several column blocks: o_t in fp32 [T, H*dv]
+  float* raw;                     // FORMs 1, 2, several column blocks: o_t in fp32 [T, H*dv]
   int H, d, dv, cw;               // cw: state columns per workgroup
+  int ldd;                        // stride of decays (FORM 2 reads a table of powers)
+  const float* table; int rot;    // FORM 2: [T, rot] cosines | sines
 };
 
 template <typename S, int D, int P, int FORM>
@@ -86,7 +92,7 @@ __global__ void __launch_bounds__(1024) scalar_recurrence_kernel(ScalarRecArgs a
   const int slot = a.slots[s];
   const int t0 = a.cu[s], t1 = a.cu[s + 1];
   const int c = threadIdx.x % dvp, part = threadIdx.x / dvp;
-  const bool fused_norm = FORM == 1 && a.raw == nullptr;
+  const bool fused_norm = FORM != 0 && a.raw == nullptr;
   if (slot < 0) {
     for (int t = t0; t < t1; ++t)
       if (c < ncol && part == 0) {
@@ -115,6 +121,7 @@ __global__ void __launch_bounds__(1024) scalar_recurrence_kernel(ScalarRecArgs a
     for (int i = threadIdx.x; i < d; i += blockDim.x) nvec[i] = fresh ? 0.f : np[i];
   }
   const float qscale = FORM == 1 ? 1.f / sqrtf((float)d) : 1.f;
+  const float kscale = FORM == 2 ? 1.f / sqrtf((float)d) : 1.f;
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, nw = blockDim.x >> 6;
   const int voff = 2 * H * d + h * dv + c0, goff = 2 * H * d + H * dv + h * dv + c0;
   const int ioff = 2 * H * d + 2 * H * dv + h, foff = ioff + H;
@@ -134,12 +141,24 @@ __global__ void __launch_bounds__(1024) scalar_recurrence_kernel(ScalarRecArgs a
     const int dd = D ? D : d;
     for (int i = threadIdx.x; i < n * dd; i += blockDim.x) {
       const float* row = a.proj + (long)(tc + i / dd) * a.ldp + h * dd + i % dd;
-      const float q = row[0], k = row[H * dd];
+      float q = row[0], k = row[H * dd];
+      if (FORM == 2) {
+        const int c2 = i % dd, hr = a.rot >> 1;
+        if (c2 < a.rot) {
+          const bool second = c2 >= hr;
+          const int ci = second ? c2 - hr : c2, po = second ? -hr : hr;
+          const float* tb = a.table + (long)(tc + i / dd) * a.rot;
+          const float cs = tb[ci], sn = second ? tb[hr + ci] : -tb[hr + ci];
+          q = q * cs + row[po] * sn;
+          k = k * cs + row[H * dd + po] * sn;
+        }
+        k *= kscale;
+      }
       qv[i] = FORM == 0 ? silu32(q) : q * qscale;
       kv[i] = FORM == 0 ? silu32(k) : k;
     }
-    if (FORM == 0) {
-      if (threadIdx.x < n) { ab[2 * threadIdx.x] = a.decays[h]; ab[2 * threadIdx.x + 1] = 1.f; }
+    if (FORM != 1) {
+      if (threadIdx.x < n) { ab[2 * threadIdx.x] = a.decays[(long)h * a.ldd]; ab[2 * threadIdx.x + 1] = 1.f; }
     } else {
       if (threadIdx.x < n) {                   // the gates' logarithms, a token a thread
         const float* row = a.proj + (long)(tc + threadIdx.x) * a.ldp;
@@ -237,7 +256,7 @@ __global__ void __launch_bounds__(1024) scalar_recurrence_kernel(ScalarRecArgs a
           ((float*)a.out)[t * a.ldo + h * dv + c0 + k] = o;
         }
       } else {
-        const float inv = 1.f / den[tt];
+        const float inv = FORM == 1 ? 1.f / den[tt] : 1.f;
         float ss = 0.f;
         for (int k = lane; k < ncol; k += 64) {
           float o = ov[tt * dvp + k];
@@ -252,6 +271,10 @@ __global__ void __launch_bounds__(1024) scalar_recurrence_kernel(ScalarRecArgs a
         const float rs = 1.f / sqrtf(ss / (float)dv + a.eps);
         for (int k = lane; k < ncol; k += 64) {
           const float g = a.proj[t * a.ldp + goff + k];
+          if (FORM == 2) {
+            stf((S*)a.out + t * a.ldo + h * dv + k, ov[tt * dvp + k] * rs * silu32(g));
+            continue;
+          }
           const float val = ov[tt * dvp + k] * rs * ldf((const S*)a.norm_w + h * dv + k) *
                             (1.f / (1.f + expf(-g))) * a.out_scale;
           stf((S*)a.out + t * a.ldo + h * dv + k, val);
@@ -327,7 +350,7 @@ extern "C" int dli_scalar_recurrence(const float* proj, int ldp, int form, const
     return (int)hipErrorInvalidValue;
   if (cw == 0 || cw >= dv) { cw = dv; raw = form == 1 ? nullptr : raw; }
   ScalarRecArgs a{proj, ldp, decays, if_b, cap, norm_w, eps, state, nstate, slots, cu, positions,
-                  out, ldo, out_scale, raw, H, d, dv, cw};
+                  out, ldo, out_scale, raw, H, d, dv, cw, 1, nullptr, 0};
   if (form == 0) {
     if (decays == nullptr || out == nullptr) return (int)hipErrorInvalidValue;
     return launch_scalar_recurrence<float, 0>(a, num_seqs, st);
@@ -338,4 +361,16 @@ extern "C" int dli_scalar_recurrence(const float* proj, int ldp, int form, const
   if (dt == 0) return launch_scalar_recurrence<u16, 1>(a, num_seqs, st);
   if (dt == 1) return launch_scalar_recurrence<float, 1>(a, num_seqs, st);
   return (int)hipErrorInvalidValue;
+}
+
+// the walk form of retention (see retention.hip, which takes long portions): decay_pow [H][ldd]
+// holds the powers of every head's decay, power 1 at column 1
+int retention_walk(const float* proj, int ldp, const float* table, int rot, const float* decay_pow,
+                   int ldd, float eps, float* state, const int* slots, const int* cu,
+                   const int* positions, void* out, int ldo, int num_seqs, int H, int d, int dv,
+                   int cw, float* raw, int dt, hipStream_t st) {
+  ScalarRecArgs a{proj, ldp, decay_pow + 1, nullptr, 0.f, nullptr, eps, state, nullptr, slots, cu,
+                  positions, out, ldo, 1.f, raw, H, d, dv, cw, ldd, table, rot};
+  if (dt == 0) return launch_scalar_recurrence<u16, 2>(a, num_seqs, st);
+  return launch_scalar_recurrence<float, 2>(a, num_seqs, st);
 }

@@ -15,6 +15,8 @@
 //  * sink    != null: exp(sink[h]) joins head h's softmax denominator: a key with that score
 //                     and no value, counted once (the running max / sum start from it)
 //  * out_scale:       the output is multiplied by it
+//  * keep_first: positions below it stay visible past the window. The visible keys of a query
+//                     are then two runs, [0, keep) and [lo, p], walked as one list of indices
 //  * chunk   > 0: a query also sees only the keys of its own block of `chunk` positions
 //                     (blocks counted from position 0 of the sequence)
 //  * Gk != G: the key rows hold Gk heads of dq while the values hold G heads of dv (Gk = 1:
@@ -59,6 +61,7 @@ struct WinAttnArgs {
   int Gk, chunk;
   const float* sink;                    // [H] or null
   int head_gate; float out_scale;
+  int keep_first;
 };
 
 template <typename S>
@@ -77,7 +80,8 @@ __global__ void __launch_bounds__(256) window_attention_kernel(WinAttnArgs a) {
   const int p = a.positions[t];
   int lo = max(0, p - a.window + 1);
   if (a.chunk > 0) lo = max(lo, p / a.chunk * a.chunk);
-  const int n = p + 1 - lo;
+  const int kf = min(a.keep_first, lo);      // kept keys before the window
+  const int n = kf + p + 1 - lo, skip = lo - kf;   // list index i >= kf is key i + skip
   const int tid = threadIdx.x;
   const S* qrow = (const S*)a.q + (long)t * a.ldq;
   for (int i = tid; i < H * dq; i += blockDim.x) qs[i] = ldf(qrow + i);
@@ -94,10 +98,10 @@ __global__ void __launch_bounds__(256) window_attention_kernel(WinAttnArgs a) {
 
   for (int pass = 0; pass < 2; ++pass) {
     for (int tile = 0; tile < ntiles; ++tile) {
-      const int j0 = lo + tile * KT;
+      const int i0 = tile * KT;
       __syncthreads();
       if (tid < KT) {
-        const int j = j0 + tid;
+        const int j = i0 + tid < kf ? i0 + tid : i0 + tid + skip;
         slot[tid] = j <= p ? bt[j / a.block_size] * a.block_size + j % a.block_size : -1;
       }
       __syncthreads();
@@ -111,7 +115,7 @@ __global__ void __launch_bounds__(256) window_attention_kernel(WinAttnArgs a) {
           float d0 = 0.f;
           for (int c = 0; c < dq; ++c) d0 += qh[c] * ldf(kr + c);
           sc = d0 * a.scale;
-          if (a.slopes != nullptr) sc -= a.slopes[h] * (float)(p - (j0 + jj));
+          if (a.slopes != nullptr) sc -= a.slopes[h] * (float)(p - (i0 + jj < kf ? i0 + jj : i0 + jj + skip));
         }
         pt[idx] = sc;
       }
@@ -148,7 +152,7 @@ __global__ void __launch_bounds__(256) window_attention_kernel(WinAttnArgs a) {
           __syncthreads();
           wts = mx;
         }
-        const int kmax = min(KT, p + 1 - j0);
+        const int kmax = min(KT, n - i0);
 #pragma unroll
         for (int i = 0; i < MAX_ACC; ++i) {
           const int o = tid + i * 256;
@@ -184,10 +188,10 @@ extern "C" int dli_window_attention(
     int ldo, const float* gate, int ldg, const float* slopes, const float* talk, const int* cu,
     const int* positions, const int* block_tables, int bt_stride, int block_size, int num_seqs,
     int max_seqlen, int H, int G, int dq, int dv, int window, float scale, int Gk, int chunk,
-    const float* sink, int head_gate, float out_scale, int dt, hipStream_t st) {
+    const float* sink, int head_gate, float out_scale, int keep_first, int dt, hipStream_t st) {
   if (num_seqs <= 0 || max_seqlen <= 0) return 0;
   if (H < 1 || G < 1 || H % G || Gk < 1 || H % Gk || chunk < 0 || dq < 1 || dv < 1 ||
-      window < 1 || block_size < 1 ||
+      window < 1 || block_size < 1 || keep_first < 0 || (keep_first > 0 && chunk > 0) ||
       (long)H * dv > 256L * MAX_ACC)
     return (int)hipErrorInvalidValue;
   const size_t sh = ((size_t)H * dq + 2 * (size_t)H * KT + 2 * H + KT) * 4;
@@ -205,7 +209,7 @@ extern "C" int dli_window_attention(
   }
   WinAttnArgs a{q, ldq, k, k_stride, v, v_stride, out, ldo, gate, ldg, slopes, talk, cu,
                 positions, block_tables, bt_stride, block_size, H, G, dq, dv, window, scale,
-                Gk, chunk, sink, head_gate, out_scale};
+                Gk, chunk, sink, head_gate, out_scale, keep_first};
   dim3 grid(max_seqlen, num_seqs);
   if (dt == 0) window_attention_kernel<u16><<<grid, 256, sh, st>>>(a);
   else if (dt == 1) window_attention_kernel<float><<<grid, 256, sh, st>>>(a);

@@ -76,6 +76,9 @@ struct MfmaArgs {
   // from (sink, 1) instead of (-inf, 0). head_gate: the gate row holds one number per head.
   // out_scale multiplies the output.
   const float* sink; int head_gate; float out_scale;
+  // > 0: positions below it stay visible past the window. A tile's keys are then two runs, [0,
+  // keep) and [lo, last], walked as one list of indices
+  int keep_first;
   // value slice of a workgroup: 128 with all heads in it; in the wide form the whole value
   // width up to 512 (narrower values take a narrower LDS image, so more workgroups share a CU)
   int dvw;
@@ -130,7 +133,9 @@ __global__ void __launch_bounds__(512) window_attention_mfma_kernel(MfmaArgs a) 
   const int p_last = a.rowmul > 1 ? p0 : p0 + nq - 1;
   // the first query's lower bound is the lowest of the tile (window and block alike)
   const int lo = max(max(0, p0 - a.window + 1), a.chunk > 0 ? p0 / a.chunk * a.chunk : 0);
-  const int ntiles = (p_last - lo) / TK + 1;
+  // kept keys before the window of the tile's first query; list index i >= kf is key i + skip
+  const int kf = min(a.keep_first, lo), skip = lo - kf;
+  const int ntiles = (p_last - skip) / TK + 1;
   const int* bt = a.block_tables + (long)s * a.bt_stride;
   const bool rgrp = a.vrows > 0;
   const int hpg = rgrp ? 1 : H / G, Gk = a.Gk, hpk = H / Gk;
@@ -231,19 +236,19 @@ __global__ void __launch_bounds__(512) window_attention_mfma_kernel(MfmaArgs a) 
   const bool slots_once = a.slot_cap >= ntiles * TK;
   if (slots_once) {
     for (int i = tid + tile_lo * TK; i < tile_hi * TK; i += 512) {
-      const int j = lo + i;
+      const int j = i < kf ? i : i + skip;
       slot_all[i] = j <= p_last ? bt[j / a.block_size] * a.block_size + j % a.block_size : -1;
     }
   }
 
   for (int pass = pass_lo; pass < pass_hi; ++pass) {
     for (int tile = tile_lo; tile < tile_hi; ++tile) {
-      const int j0 = lo + tile * TK;
+      const int i0 = tile * TK, j0 = i0 + skip;     // j0: the tile's first key past the kept ones
       int* slot = slots_once ? slot_all + tile * TK : slot_all;
       if (!slots_once) {
         __syncthreads();                          // previous tile's readers are done
         if (tid < TK) {
-          const int j = j0 + tid;
+          const int j = i0 + tid < kf ? i0 + tid : j0 + tid;
           slot[tid] = j <= p_last ? bt[j / a.block_size] * a.block_size + j % a.block_size : -1;
         }
       }
@@ -333,7 +338,7 @@ __global__ void __launch_bounds__(512) window_attention_mfma_kernel(MfmaArgs a) 
           float sv[8];
           float tmax = -INFINITY;
           // interior tiles (every key visible to every query row): no masking arithmetic
-          const bool interior = nq == TQ && j0 + TK - 1 <= p0 && j0 > p_last - a.window &&
+          const bool interior = nq == TQ && i0 >= kf && j0 + TK - 1 <= p0 && j0 > p_last - a.window &&
                                 j0 >= clo_last;
 #pragma unroll
           for (int kb = 0; kb < 2; ++kb)
@@ -341,9 +346,11 @@ __global__ void __launch_bounds__(512) window_attention_mfma_kernel(MfmaArgs a) 
             for (int r = 0; r < 4; ++r) {
               float x = fmaf(sacc[kb][r], scale2, b0 + slope2 * (float)(kb * 16 + r));
               if (!interior) {
-                const int key = j0 + kb * 16 + fq * 4 + r;
+                const int ki = i0 + kb * 16 + fq * 4 + r;
+                const int key = ki < kf ? ki : ki + skip;
                 const int dist = my_p - key;
-                if (!my_q || dist < 0 || dist >= a.window || key < my_clo) x = -INFINITY;
+                if (!my_q || dist < 0 || (dist >= a.window && key >= a.keep_first) || key < my_clo)
+                  x = -INFINITY;
               }
               sv[kb * 4 + r] = x;
               tmax = fmaxf(tmax, x);
@@ -651,14 +658,16 @@ extern "C" int dli_window_attention_mfma(
     const int* positions, const int* block_tables, int bt_stride, int block_size, int num_seqs,
     int max_seqlen, int H, int G, int dq, int dv, int window, float scale, int T, void* ws,
     int rowhead, int Gk, int chunk, const float* sink, int head_gate, float out_scale,
-    hipStream_t st) {
+    int keep_first, hipStream_t st) {
   if (num_seqs <= 0 || max_seqlen <= 0) return 0;
   if (chunk < 0 || Gk < 1) return (int)hipErrorInvalidValue;
   // the sink rides on the one-pass forms' running (max, sum); with head mixing it has no place
   if (sink != nullptr && (talk != nullptr || rowhead)) return (int)hipErrorNotSupported;
   if (head_gate && dv % 4) return (int)hipErrorNotSupported;
   // keys a query tile can see: bounds the slot table and the key splits
-  const int weff = chunk > 0 && chunk < window ? chunk : window;
+  if (keep_first < 0 || (keep_first > 0 && (chunk > 0 || slopes != nullptr)))
+    return (int)hipErrorInvalidValue;
+  const int weff = (chunk > 0 && chunk < window ? chunk : window) + keep_first;
   int rowmul = 1, vrows = 0;
   if (rowhead) {
     if (talk != nullptr || gate != nullptr || slopes != nullptr || Gk != 1 || G < 1 || H % G ||
@@ -734,7 +743,7 @@ extern "C" int dli_window_attention_mfma(
   MfmaArgs a{(const u16*)q, ldq, (const u16*)k, k_stride, (const u16*)v, v_stride, (u16*)out,
              ldo, gate, ldg, slopes, talk, cu, positions, block_tables, bt_stride, block_size,
              H, G, dq, dv, window, scale, Gk, chunk, Hp, CG, 0, 1, ndvs, wide ? 1 : 0, nhs, rowmul,
-             vrows, cgv, slot_cap, sink, head_gate, out_scale, dvw, nullptr, nullptr, 0};
+             vrows, cgv, slot_cap, sink, head_gate, out_scale, keep_first, dvw, nullptr, nullptr, 0};
   if (nsplit == 1) {
     dim3 grid(qtiles, num_seqs, ndvs * nhs);
     WA_LAUNCH(grid);

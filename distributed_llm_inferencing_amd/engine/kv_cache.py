@@ -98,7 +98,10 @@ class HybridCache:
                             with ``kv_from`` gets the tensors of that layer's run (it writes
                             nothing)
 
-    * ``lightning``:        (state [state_slots, H, d, dv] fp32,)
+    * ``lightning``, ``retention``: (state [state_slots, H, d, dv] fp32,)
+    * ``rope_attention``:   (k [slots, G*d], v [slots, G*dv])   rotated keys and values (the
+                            unrotated keys when values are tied to them; without any rotation
+                            the two are one tensor)
     * ``parallel``:         (k [slots, G*d], v [slots, G*dv], state [state_slots, Hr, dr, dvr]
                             fp32, nm [state_slots, Hr, dr + 1] fp32): the attention side's
                             normed, rotated keys and values; the memory side's matrix, and its
@@ -146,6 +149,10 @@ class HybridCache:
             if s.kind == "attention":
                 e = (torch.zeros(rows, s.kv_heads * s.dim, dtype=dtype, device=device),
                      torch.zeros(rows, s.kv_heads * s.dim, dtype=dtype, device=device))
+            elif s.kind == "rope_attention":
+                k = torch.zeros(rows, s.kv_heads * s.dim, dtype=dtype, device=device)
+                e = (k, k if s.tied_values and not s.rot_dims else
+                     torch.zeros(rows, s.kv_heads * s.vdim, dtype=dtype, device=device))
             elif s.kind == "latent_attention":
                 e = (torch.zeros(rows, s.kv_rank + s.rot_dim, dtype=dtype, device=device),)
             elif s.kind == "parallel":

@@ -30,12 +30,19 @@ class LayerSpec:
     the queries through an RMS-normed latent of that width, ``head_gate`` multiplies each
     head's output by one sigmoid gate, ``rot_half`` pairs rotated dimension i with i +
     rot_dims/2 instead of (2i, 2i+1), and ``kv_from`` reads another layer's cached latent.
+    ``retention`` (linear attention with one fixed decay per head over rotated queries and keys,
+    each head's read-out divided by its own RMS, SiLU output gate) and ``rope_attention``
+    (grouped-query softmax attention over ``window`` positions plus the first ``keep_first``
+    ones, the first ``rot_dims`` dims of q and k rotated; ``bias``: q / k / v / output
+    projections carry biases; ``tied_values``: the values are the keys before their rotation).
 
     feed-forward kinds (``ff_kind``): ``gated_gelu`` (down(gelu(gate) * up)), ``gelu``
     (down(gelu(up))) and ``moe`` (``experts`` gated-SiLU experts of width ``ff`` plus
     ``identity`` pass-through experts, ``top`` per token chosen by softmax score + a learned
     correction and weighted by the un-renormalised score, and a shared expert of width
-    ``shared_ff`` behind a per-token sigmoid gate) and ``gated_silu`` (down(silu(gate) * up)).
+    ``shared_ff`` behind a per-token sigmoid gate), ``gated_silu`` (down(silu(gate) * up)) and
+    ``clamp_swish`` (down(g sigmoid(1.702 g) (u + 1)), g = min(gate, ``act_limit``), u = up
+    clamped to +-``act_limit``).
     A mixture with ``router`` = ``logit_topk`` picks the ``top`` largest biased logits and
     weighs them by the softmax over the chosen ones; ``expert_act`` = ``gelu_erf`` makes the
     experts (and the shared one, then ungated) down(gelu(up)) with the exact GELU."""
@@ -76,13 +83,17 @@ class LayerSpec:
     router_groups: int = 1    # group_score router: equal groups of neighbouring experts
     router_keep: int = 1      # ... of which the best this many may be chosen from
     router_scale: float = 1.0     # ... and the chosen scores are multiplied by this
-    act_limit: float = 0.0    # clamp_swish experts: the clamp
+    act_limit: float = 0.0    # clamp_swish: the clamp
+    keep_first: int = 0       # rope_attention: these first positions stay visible past the window
+    bias: bool = False        # rope_attention: biased projections
+    tied_values: bool = False     # rope_attention: values = the keys before their rotation
 
     @property
     def has_state(self) -> bool:
         """The layer keeps something per sequence besides cache rows: a recurrent state, or
         the previous token's mixer input."""
-        return self.kind in ("hgrn2", "gla", "lightning", "parallel", "mlstm") or self.shift
+        return self.kind in ("hgrn2", "gla", "lightning", "parallel", "mlstm",
+                             "retention") or self.shift
 
     @classmethod
     def from_dict(cls, d: dict) -> "LayerSpec":
@@ -101,7 +112,7 @@ class ModelConfig:
     name: str
     arch: str                 # "llama" (llama / mixtral family), "gpt2", or a hybrid
                               # (layer-list) design: "buborax", "pulunex", "risutar",
-                              # "lapunex"
+                              # "lapunex", "bamudra"
     hidden_size: int
     num_layers: int
     num_heads: int
@@ -147,6 +158,8 @@ class ModelConfig:
     # a loop pass starts with x = W_in [x ; x0] + step[pass]; False: passes follow each other
     # with nothing in between
     loop_entry: bool = True
+    # every pass of the loop but the first starts with x = x + x0 (x0 = the embedding output)
+    loop_add: bool = False
 
     @property
     def is_hybrid(self) -> bool:
@@ -233,6 +246,8 @@ class ModelConfig:
             return 2 * s.kv_heads * s.dim           # normed keys + raw keys (the values)
         if s.kind == "latent_attention":
             return 0 if s.kv_from >= 0 else s.kv_rank + s.rot_dim
+        if s.kind == "rope_attention":
+            return s.kv_heads * (s.dim + s.vdim)
         if s.kind == "talk_attention":
             return 0 if s.kv_from >= 0 else s.kv_heads * (s.dim + s.vdim)
         if s.kind == "parallel":
@@ -387,10 +402,25 @@ LAPUNEX_TINY = hybrid_config(
     loop=(0, 2, 2), norm_eps=1e-5, embed_scale=6.0, streams=2, norm_offset=1.0,
     loop_entry=False)
 
+_BAMUDRA_RETENTION = LayerSpec("retention", heads=3, dim=32, vdim=48, rot_dims=16, rot_base=4000.0,
+                               decays=(0.9, 0.97, 0.995))
+
+# Bamudra at test size: retention layers with and without feed-forward, windowed attention with
+# kept first tokens over tied keys and values, a loop that re-adds the embedding
+BAMUDRA_TINY = hybrid_config(
+    "bamudra-tiny", width=128, vocab=384, arch="bamudra",
+    layer_specs=(
+        LayerSpec("rope_attention", heads=4, kv_heads=2, dim=32, vdim=32, window=24, keep_first=3,
+                  scale=0.18, rot_dims=24, rot_base=3000.0, bias=True, tied_values=True, ff=192,
+                  ff_kind="clamp_swish", act_limit=2.0),
+        _BAMUDRA_RETENTION,
+        replace(_BAMUDRA_RETENTION, ff=160, ff_kind="clamp_swish", act_limit=1.0)),
+    loop=(1, 3, 2), norm_eps=1e-5, loop_entry=False, loop_add=True)
+
 _REGISTRY = {c.name: c for c in
              (GPT2, LLAMA3_8B, LLAMA3_70B, MIXTRAL_8X7B, LLAMA_TINY, LLAMA_TINY128,
               LLAMA_TINY8, MIXTRAL_TINY, MIXTRAL_TINY8E, GPT2_TINY, BUBORAX_TINY, PULUNEX_TINY,
-              RISUTAR_TINY, LAPUNEX_TINY)}
+              RISUTAR_TINY, LAPUNEX_TINY, BAMUDRA_TINY)}
 
 _ALIASES = {
     "openai-community/gpt2": "gpt2",

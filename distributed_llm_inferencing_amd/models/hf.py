@@ -25,7 +25,7 @@ from typing import Dict, Iterable, Iterator, Optional, Tuple
 import torch
 
 from .configs import ModelConfig
-from .weights import (from_buborax_state_dict, from_hf_state_dict, from_lapunex_state_dict,
+from .weights import (from_bamudra_state_dict, from_buborax_state_dict, from_hf_state_dict, from_lapunex_state_dict,
                       from_pulunex_state_dict, from_risutar_state_dict)
 
 
@@ -59,7 +59,7 @@ def find_hf_dir(root: str, name: str) -> Optional[Path]:
     return None
 
 
-NATIVE_ARCHS = ("Buborax", "Pulunex", "Risutar", "Lapunex")
+NATIVE_ARCHS = ("Buborax", "Pulunex", "Risutar", "Lapunex", "Bamudra")
 
 
 def buborax_config(c: dict, name: Optional[str] = None) -> ModelConfig:
@@ -300,9 +300,61 @@ def lapunex_config(c: dict, name: Optional[str] = None) -> ModelConfig:
                          streams=int(c.get("streams") or 0), norm_offset=1.0, loop_entry=False)
 
 
+def bamudra_config(c: dict, name: Optional[str] = None) -> ModelConfig:
+    """A Bamudra ``config.json``: ``width``, ``vocab``, ``norm`` {eps}, ``loop`` {start, stop,
+    times} (optional) and ``layers``, a list of {type, mixer, mlp}: type ``retention`` with mixer
+    {heads, dim, vdim, decay [per head], rot {base, dims}} or ``attention`` with mixer {heads,
+    kv_heads, dim, vdim, scale, rot {base, dims}, mask {size, keep_first}}; mlp null or {kind:
+    dense, ff, limit}. Every size and constant is read from it."""
+    from .configs import LayerSpec, hybrid_config
+    specs = []
+    for i, L in enumerate(c["layers"]):
+        mx, kind = L["mixer"], L["type"]
+        ff = dict(ff=0)
+        mlp = L.get("mlp")
+        if mlp:
+            if mlp.get("kind", "dense") != "dense":
+                raise ValueError(f"unsupported feed-forward kind '{mlp.get('kind')}'")
+            ff = dict(ff=int(mlp["ff"]), ff_kind="clamp_swish", act_limit=float(mlp["limit"]))
+        H, d = int(mx["heads"]), int(mx["dim"])
+        dv = int(mx.get("vdim", d))
+        rot = mx.get("rot") or {}
+        dims = int(rot.get("dims") or 0)
+        if dims % 2 or dims > d:
+            raise ValueError(f"layer {i}: rot.dims {dims} of a head of {d}")
+        ff.update(rot_dims=dims, rot_base=float(rot.get("base", 10000.0)))
+        if kind == "retention":
+            decays = tuple(float(a) for a in mx["decay"])
+            if len(decays) != H:
+                raise ValueError(f"layer {i}: {len(decays)} decays for {H} heads")
+            specs.append(LayerSpec("retention", heads=H, dim=d, vdim=dv, decays=decays, **ff))
+        elif kind == "attention":
+            G = int(mx.get("kv_heads") or H)
+            if H % G or dv != d:
+                raise ValueError(f"layer {i}: the values are the keys (vdim == dim) and heads "
+                                 "must be a multiple of kv_heads")
+            mask = mx.get("mask") or {}
+            specs.append(LayerSpec("rope_attention", heads=H, kv_heads=G, dim=d, vdim=dv,
+                                   window=int(mask.get("size") or (1 << 30)),
+                                   keep_first=int(mask.get("keep_first") or 0),
+                                   scale=float(mx.get("scale", d ** -0.5)), bias=True,
+                                   tied_values=True, **ff))
+        else:
+            raise ValueError(f"unsupported mixer type '{kind}'")
+    lp = c.get("loop")
+    loop = (int(lp["start"]), int(lp["stop"]), int(lp["times"])) if lp else ()
+    if loop and not (0 <= loop[0] < loop[1] <= len(specs) and loop[2] >= 1):
+        raise ValueError(f"bad loop {loop} for {len(specs)} layers")
+    return hybrid_config(name or c.get("_name_or_path") or "bamudra", int(c["width"]),
+                         int(c["vocab"]), specs, loop,
+                         norm_eps=float((c.get("norm") or {}).get("eps", 1e-5)), arch="bamudra",
+                         loop_entry=False, loop_add=bool(loop))
+
+
 def config_from_hf(c: dict, name: Optional[str] = None) -> ModelConfig:
     """Map a ``config.json``: HF llama / mistral / mixtral / gpt2 model types, or one of the
-    native layer-list designs (``architecture``: Buborax, Pulunex, Risutar, Lapunex)."""
+    native layer-list designs (``architecture``: Buborax, Pulunex, Risutar, Lapunex,
+    Bamudra)."""
     if c.get("architecture") == "Buborax":
         return buborax_config(c, name)
     if c.get("architecture") == "Pulunex":
@@ -311,6 +363,8 @@ def config_from_hf(c: dict, name: Optional[str] = None) -> ModelConfig:
         return risutar_config(c, name)
     if c.get("architecture") == "Lapunex":
         return lapunex_config(c, name)
+    if c.get("architecture") == "Bamudra":
+        return bamudra_config(c, name)
     mt = c.get("model_type", "")
     name = name or c.get("_name_or_path") or mt
     if mt == "gpt2":
@@ -426,6 +480,8 @@ def load_hf_dir(d, device="cpu", dtype=torch.bfloat16, name: Optional[str] = Non
             cfg, params = from_risutar_state_dict(cfg, sd, dtype=dtype)
         elif cfg.arch == "lapunex":
             params = from_lapunex_state_dict(cfg, sd, dtype=dtype)
+        elif cfg.arch == "bamudra":
+            params = from_bamudra_state_dict(cfg, sd, dtype=dtype)
         elif cfg.is_hybrid:
             params = from_buborax_state_dict(cfg, sd, dtype=dtype)
         else:

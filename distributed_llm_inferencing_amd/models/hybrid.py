@@ -1,7 +1,7 @@
-"""Hybrid decoder (archs ``buborax``, ``pulunex``, ``risutar``, ``lapunex``): a layer list that
-mixes windowed attention, latent attention, gated linear recurrences (HGRN2, gated linear
-attention, fixed-decay linear attention, a matrix memory beside a sink attention) and block
-attention with head-mixed scores; dense, gated and routed feed-forwards; a shared-weight loop,
+"""Hybrid decoder (archs ``buborax``, ``pulunex``, ``risutar``, ``lapunex``, ``bamudra``): a
+layer list that mixes windowed attention, latent attention, gated linear recurrences (HGRN2,
+gated linear attention, fixed-decay linear attention with or without rotation, a matrix memory
+beside a sink attention) and block attention with head-mixed scores; dense, gated and routed feed-forwards; a shared-weight loop,
 grouped RMS norms, token shift and an fp32 residual stream (or several hyper-connected
 streams) — served by the same engine, scheduler, block manager and runner as the transformer
 families.
@@ -28,8 +28,9 @@ and the final norm reads the sum of the streams (``ops.hybrid.hyper_mix`` fuses 
 write-back with the next sublayer's read and norm).
 
 * Layers [start, stop) of the loop run ``times`` times with the same weights; a pass starts
-  with x = W_in [x ; x0] + step[pass] (x0 = the embedding output). Every run owns its cache or
-  state (``engine.kv_cache.HybridCache``).
+  with x = W_in [x ; x0] + step[pass] (x0 = the embedding output), or every pass but the first
+  with x = x + x0 (``cfg.loop_add``). Every run owns its cache or state
+  (``engine.kv_cache.HybridCache``).
 * The residual stream and every norm are fp32; GEMM operands use the storage dtype of the
   weights (bf16 when serving; fp32 weights give an all-fp32 model). Each residual add is fused
   with the norm that follows it (``ops.hybrid.resadd_groupnorm``).
@@ -60,6 +61,9 @@ class HybridLM(TransformerLM):
         if layer_start != 0 or (layer_end is not None and layer_end != cfg.num_layers):
             raise ValueError("hybrid designs run on one stage (the loop entry reads the "
                              "embedding output)")
+        if any(s.bias for s in cfg.layer_specs) and (cfg.residual_mult != 1.0 or cfg.streams
+                                                     or cfg.post_norm):
+            raise ValueError("output biases ride on the plain residual add (multiplier 1)")
         for i, spec in enumerate(cfg.layer_specs):
             prepare_feed_forward(spec, params, f"layers.{i}.")
         super().__init__(cfg, params, 0, None, device)
@@ -178,34 +182,39 @@ class HybridLM(TransformerLM):
         eps, groups, m, off = cfg.norm_eps, cfg.norm_groups, cfg.residual_mult, cfg.norm_offset
         step = self._step_view(b, kv_caches.block_size)
         entries = kv_caches.entries
-        x0 = x.clone() if cfg.loop and cfg.loop_entry else None
-        pending = None                      # a sub-block's fp32 output awaiting its add
+        x0 = x.clone() if cfg.loop and (cfg.loop_entry or cfg.loop_add) else None
+        pending = bias = None               # a sub-block's fp32 output (and bias) awaiting its add
         for ri, (li, t, first) in enumerate(self.runs):
             spec, lp = cfg.layer_specs[li], self.layers[li]
             if first:
                 if pending is not None:
-                    H.resadd_groupnorm(x, pending, None, groups, eps, mult=m)
-                    pending = None
+                    H.resadd_groupnorm(x, pending, None, groups, eps, mult=m, bias=bias)
+                    pending = bias = None
                 y = H.linear_any(H.concat_cast(x, x0, self.dtype), p["loop_in"])
                 h = H.resadd_groupnorm(x, y, lp["norm1"], groups, eps, mult=1.0, keep=0.0,
                                        bias=p["loop_step"][t], out_f32=spec.shift)
             else:
-                h = H.resadd_groupnorm(x, pending, lp["norm1"], groups, eps, mult=m,
-                                       out_f32=spec.shift, w_offset=off)
+                # a later pass of an adding loop starts with the embedding output on top
+                again = cfg.loop_add and t > 0 and li == cfg.loop[0]
+                h = H.resadd_groupnorm(x, pending, lp["norm1"], groups, eps, mult=m, bias=bias,
+                                       out_f32=spec.shift, w_offset=off,
+                                       add=x0 if again else None)
             if spec.shift:                  # the mixer reads the rows mixed with their predecessors
                 h = H.token_shift(h, lp["shift"], kv_caches.shift_states[ri], step.state_slots,
                                   step.cu_seqlens, step.max_seqlen, step.positions)
             y = MIXERS[spec.kind](spec, lp, h, step, entries[ri], eps)
+            bias = lp.get("b_out")          # the output projection's bias rides on the add
             if spec.ff:
-                h = H.resadd_groupnorm(x, y, lp["norm2"], groups, eps, mult=m, w_offset=off)
-                y = FEED_FORWARDS[spec.ff_kind](spec, lp, h)
+                h = H.resadd_groupnorm(x, y, lp["norm2"], groups, eps, mult=m, w_offset=off,
+                                       bias=bias)
+                y, bias = FEED_FORWARDS[spec.ff_kind](spec, lp, h), None
             pending = y
             if self.layer_trace is not None:
-                H.resadd_groupnorm(x, pending, None, groups, eps, mult=m)
-                pending = None
+                H.resadd_groupnorm(x, pending, None, groups, eps, mult=m, bias=bias)
+                pending = bias = None
                 self.layer_trace.append(x.clone())
         if pending is not None:
-            H.resadd_groupnorm(x, pending, None, groups, eps, mult=m)
+            H.resadd_groupnorm(x, pending, None, groups, eps, mult=m, bias=bias)
         return x
 
     def final_hidden(self, hidden: torch.Tensor, b: DeviceBatch) -> torch.Tensor:

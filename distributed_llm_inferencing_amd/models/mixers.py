@@ -12,7 +12,7 @@ derived at load time (``derive_constants``); ``step``: the per-step metadata (``
 """
 from __future__ import annotations
 
-from dataclasses import dataclass
+from dataclasses import dataclass, field
 from typing import Optional
 
 import torch
@@ -33,6 +33,18 @@ class StepView:
     block_size: int
     state_slots: Optional[torch.Tensor]   # [S] int32 recurrent-state slot (-1: padding row)
     max_context: int = 1 << 30      # no position of this step is at or beyond this
+    tables: dict = field(default_factory=dict)      # rotation tables made so far in this step
+
+    def rotation(self, spec: LayerSpec, lp: dict):
+        """fp32 [T, rot_dims] = cosines | sines of the step's positions, made once per step for
+        all layers that rotate alike; None without rotation."""
+        if not spec.rot_dims:
+            return None
+        key = (spec.rot_dims, spec.rot_base)
+        t = self.tables.get(key)
+        if t is None:
+            t = self.tables[key] = H.rotation_table(self.positions, lp["rot_freq"])
+        return t
 
 
 def derive_constants(spec: LayerSpec, lp: dict, device) -> None:
@@ -50,6 +62,13 @@ def derive_constants(spec: LayerSpec, lp: dict, device) -> None:
         lp["talk"] = lp["talk"].float().contiguous()
     elif spec.kind == "lightning":
         lp["decays"] = torch.tensor(spec.decays, dtype=torch.float64).float().to(device)
+    elif spec.kind in ("retention", "rope_attention"):
+        lp["rot_freq"] = yarn_frequencies(spec.rot_dims, spec.rot_base)[0].to(device)
+        if spec.kind == "retention":
+            # powers 0 .. RETENTION_CHUNK of every head's decay, each rounded once
+            n = torch.arange(H.RETENTION_CHUNK + 1, dtype=torch.float64)
+            dec = torch.tensor(spec.decays, dtype=torch.float64)
+            lp["decay_pow"] = torch.pow(dec[:, None], n[None, :]).float().contiguous().to(device)
     elif spec.kind == "parallel":
         freq, mscale = yarn_frequencies(spec.left.rot_dims, spec.left.rot_base,
                                         spec.left.rot_scaling)
@@ -226,9 +245,41 @@ def parallel_mixer(spec: LayerSpec, lp: dict, h, step: StepView, cache, eps: flo
     return H.linear_any(o, lp["wo"])
 
 
+def retention_mixer(spec: LayerSpec, lp: dict, h, step: StepView, cache, eps: float):
+    """Linear attention with one fixed decay per head over rotated queries and keys (no
+    activation), each head's read-out divided by its own RMS, SiLU output gate. Rotation, state,
+    norm and gate in fp32."""
+    (state,) = cache
+    proj = H.linear_any(h, lp["w_in"])                       # fp32 [T, q | k | v | gate]
+    o = H.retention(proj, step.rotation(spec, lp), spec.rot_dims, lp["decay_pow"], eps, state,
+                    step.state_slots, step.cu_seqlens, step.max_seqlen, step.positions,
+                    spec.heads, spec.dim, spec.vdim, h.dtype)
+    return H.linear_any(o, lp["wo"])
+
+
+def rope_attention_mixer(spec: LayerSpec, lp: dict, h, step: StepView, cache, eps: float):
+    """Grouped-query softmax attention over a sliding window plus kept first positions, partly
+    rotated q and k, optional biases, values optionally tied to the unrotated keys. The output
+    projection's bias is added with the residual (``HybridLM.forward_layers``)."""
+    kc, vc = cache
+    proj = H.linear_any(h, lp["w_in"])                       # fp32 [T, q | k (| v)]
+    q = H.rope_prepare(proj, lp.get("b_in"), step.rotation(spec, lp), spec.rot_dims, spec.heads,
+                       spec.kv_heads, spec.dim, spec.vdim, kc, vc, step.slot_mapping, h.dtype,
+                       spec.tied_values)
+    # a window no shorter than the step's longest context masks nothing
+    ctx = max(1, step.max_context)
+    win = min(spec.window, ctx)
+    o = H.window_attention(q, kc, vc, spec.dim, spec.vdim, spec.heads, spec.kv_heads,
+                           step.cu_seqlens, step.max_seqlen, step.positions, step.block_tables,
+                           step.block_size, win, spec.scale,
+                           keep_first=min(spec.keep_first, ctx) if win < ctx else 0)
+    return H.linear_any(o, lp["wo"])
+
+
 MIXERS = {"attention": attention_mixer, "hgrn2": hgrn2_mixer,
           "latent_attention": latent_attention_mixer, "talk_attention": talk_attention_mixer,
-          "gla": gla_mixer, "lightning": lightning_mixer, "parallel": parallel_mixer}
+          "gla": gla_mixer, "lightning": lightning_mixer, "parallel": parallel_mixer,
+          "retention": retention_mixer, "rope_attention": rope_attention_mixer}
 
 
 # ----------------------------------------------------------------------------- feed-forwards
@@ -289,6 +340,13 @@ def gated_silu_ff(spec: LayerSpec, lp: dict, h):
     return H.linear_any(act, lp["w_down"])
 
 
+def clamp_swish_ff(spec: LayerSpec, lp: dict, h):
+    """down(g sigmoid(1.702 g) (u + 1)), g = min(gate, limit), u = clamp(up, -limit, limit)."""
+    act = H.act_mul(H.linear_any(h, lp["w_gu"]), spec.ff, h.dtype, "clamp_swish",
+                    limit=spec.act_limit)
+    return H.linear_any(act, lp["w_down"])
+
+
 def moe_ff(spec: LayerSpec, lp: dict, h):
     """Routed gated-SiLU experts + identity experts + a gated shared expert, summed in fp32;
     with ``router`` = ``logit_topk``: biased logits, softmax over the chosen, ungated exact-GELU
@@ -330,4 +388,4 @@ def moe_ff(spec: LayerSpec, lp: dict, h):
 
 
 FEED_FORWARDS = {"gated_gelu": gated_gelu_ff, "gelu": gelu_ff, "moe": moe_ff,
-                 "gated_silu": gated_silu_ff}
+                 "gated_silu": gated_silu_ff, "clamp_swish": clamp_swish_ff}

@@ -64,6 +64,10 @@ def hybrid_layer_shapes(cfg: ModelConfig, i: int) -> Dict[str, tuple]:
                         wo [D, Hl*dvl + Hr*dvr] = left | right output projections
         moe, router ``group_score`` with ``clamp_swish`` experts: router [E, D],
                         w_gu [E, 2F, D], w_down [E, D, F]
+      retention:        w_in [2*H*d + 2*H*dv, D] = q | k | v | output gate, wo [D, H*dv]
+      rope_attention:   w_in [(H + G)*d (+ G*dv), D] = q | k (| v, absent with ``tied_values``),
+                        wo [D, H*dv]; with ``bias``: b_in, b_out [D]
+        clamp_swish:    w_gu [2F, D] = gate | up, w_down [D, F]
     Post-norm designs add the norms' biases norm1_b / norm2_b [D]; with a per-layer token input
     of width s: side_gate [s, D], side_proj [D, s], side_norm [D]. With hyper-connections over
     S streams every sublayer has hc1 / hc2 fp32 [S + S + S*S] = read weights | write weights |
@@ -108,6 +112,13 @@ def hybrid_layer_shapes(cfg: ModelConfig, i: int) -> Dict[str, tuple]:
                     p + "k_norm": (l.kv_heads * l.dim,), p + "sink": (l.heads,),
                     p + "o_norm": (r.heads * r.vdim,), p + "if_b": (2 * r.heads,),
                     p + "wo": (D, l.heads * l.vdim + r.heads * r.vdim)})
+    elif s.kind == "retention":
+        out.update({p + "w_in": (2 * H * (d + dv), D), p + "wo": (D, H * dv)})
+    elif s.kind == "rope_attention":
+        n_in = (H + s.kv_heads) * d + (0 if s.tied_values else s.kv_heads * dv)
+        out.update({p + "w_in": (n_in, D), p + "wo": (D, H * dv)})
+        if s.bias:
+            out.update({p + "b_in": (n_in,), p + "b_out": (D,)})
     else:
         raise ValueError(f"unknown mixer kind '{s.kind}'")
     if cfg.streams:
@@ -127,7 +138,7 @@ def hybrid_layer_shapes(cfg: ModelConfig, i: int) -> Dict[str, tuple]:
                     p + "w_up": (s.experts, s.ff, D), p + "w_down": (s.experts, D, s.ff)})
         if s.shared_ff:
             out.update({p + "ws_up": (s.shared_ff, D), p + "ws_down": (D, s.shared_ff)})
-    elif s.ff and s.ff_kind in ("gated_gelu", "gated_silu"):
+    elif s.ff and s.ff_kind in ("gated_gelu", "gated_silu", "clamp_swish"):
         out.update({p + "norm2": (D,), p + "w_gu": (2 * s.ff, D), p + "w_down": (D, s.ff)})
     elif s.ff and s.ff_kind == "gelu":
         out.update({p + "norm2": (D,), p + "w_up": (s.ff, D), p + "w_down": (D, s.ff)})
@@ -280,7 +291,7 @@ def _hybrid_init(name: str, shape: tuple, dev, dtype, seed: int) -> torch.Tensor
         return (1.0 + 2.0 * torch.randn(shape, generator=g)).to(dev, dtype)
     if name.endswith(".shift"):
         return torch.rand(shape, generator=g).to(dev, dtype)
-    if name.endswith(".b_in"):
+    if name.endswith((".b_in", ".b_out")):
         # small: a large value bias is a constant added to every token, which would make a
         # random-init router send every token to the same experts
         return (0.02 * torch.randn(shape, generator=g)).to(dev, dtype)
@@ -596,9 +607,40 @@ def from_lapunex_state_dict(cfg: ModelConfig, sd, dtype=torch.bfloat16) -> Dict[
         out[p + "w_gu"] = cv(torch.stack([torch.cat([sd[f"{f}e{e}.gate"], sd[f"{f}e{e}.up"]], 0)
                                           for e in range(s.experts)]))
         out[p + "w_down"] = cv(torch.stack([sd[f"{f}e{e}.down"] for e in range(s.experts)]))
+    return _checked(cfg, out)
+
+
+def _checked(cfg: ModelConfig, out: Dict[str, torch.Tensor]) -> Dict[str, torch.Tensor]:
+    """``out``, after every tensor's shape was compared with the configuration."""
     want = stage_param_shapes(cfg, 0, len(cfg.layer_specs), True, True)
     for k, shp in want.items():
         if k not in out or tuple(out[k].shape) != tuple(shp):
             got = tuple(out[k].shape) if k in out else None
             raise ValueError(f"{k}: the checkpoint gives {got}, the configuration {tuple(shp)}")
     return out
+
+
+# ----------------------------------------------------------------------------- Bamudra files
+def from_bamudra_state_dict(cfg: ModelConfig, sd, dtype=torch.bfloat16) -> Dict[str, torch.Tensor]:
+    """Convert a Bamudra checkpoint (tensor names ``embed``, ``head``, ``final.norm``,
+    ``l<i>.norm1|norm2``, ``l<i>.mix.q|k|v|g|o`` of a retention layer, ``l<i>.mix.q|k|o`` with
+    ``.b`` biases of an attention layer, ``l<i>.mlp.gate|up|down``; linear weights [out, in])
+    into the layout of ``hybrid_layer_shapes``: projections that read the same input are
+    stacked."""
+    cv = lambda t: t.detach().to(dtype).contiguous()  # noqa: E731
+    out = {"embed": cv(sd["embed"]), "lm_head": cv(sd["head"]), "final_norm": cv(sd["final.norm"])}
+    for i, s in enumerate(cfg.layer_specs):
+        a, p = f"l{i}.", f"layers.{i}."
+        m, f = a + "mix.", a + "mlp."
+        out[p + "norm1"] = cv(sd[a + "norm1"])
+        parts = "qkvg" if s.kind == "retention" else "qk" if s.tied_values else "qkv"
+        out[p + "w_in"] = cv(torch.cat([sd[m + n] for n in parts], 0))
+        out[p + "wo"] = cv(sd[m + "o"])
+        if s.bias:
+            out[p + "b_in"] = cv(torch.cat([sd[m + n + ".b"] for n in parts], 0))
+            out[p + "b_out"] = cv(sd[m + "o.b"])
+        if s.ff:
+            out[p + "norm2"] = cv(sd[a + "norm2"])
+            out[p + "w_gu"] = cv(torch.cat([sd[f + "gate"], sd[f + "up"]], 0))
+            out[p + "w_down"] = cv(sd[f + "down"])
+    return _checked(cfg, out)

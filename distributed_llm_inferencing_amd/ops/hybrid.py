@@ -22,6 +22,8 @@ from . import reference as R
 _call = N.call
 _p = N.ptr
 _NOT_SUPPORTED = 801            # hipErrorNotSupported: a launcher declining a shape
+# longest chunk of the retention kernels (the table of decay powers covers it)
+RETENTION_CHUNK = 64
 # DLI_WINATTN_SCALAR=1 keeps bf16 windowed attention on the scalar kernel (A/B, debugging)
 MFMA_ATTENTION = os.environ.get("DLI_WINATTN_SCALAR", "0") != "1"
 
@@ -108,8 +110,10 @@ def embedding_f32(ids: torch.Tensor, table: torch.Tensor, copy: bool = False,
 def resadd_groupnorm(x: torch.Tensor, y: Optional[torch.Tensor], w: Optional[torch.Tensor],
                      groups: int, eps: float, mult: float = 1.0, keep: float = 1.0,
                      bias: Optional[torch.Tensor] = None, dtype=None, gain: float = 1.0,
-                     out_f32: bool = False, w_offset: float = 0.0) -> Optional[torch.Tensor]:
-    """In place on the fp32 stream: x = keep * x + mult * y + bias (y, bias optional); returns
+                     out_f32: bool = False, w_offset: float = 0.0,
+                     add: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+    """In place on the fp32 stream: x = keep * x + mult * y + bias + add (y, bias and the fp32
+    rows ``add`` optional); returns
     the grouped RMS norm of the new x times ``w`` times ``gain`` in the storage dtype (None when
     w is None), or unrounded in fp32 with ``out_f32`` (what a token shift reads). ``w_offset``
     is added to the weight in fp32 (weights stored as offsets from one)."""
@@ -121,6 +125,8 @@ def resadd_groupnorm(x: torch.Tensor, y: Optional[torch.Tensor], w: Optional[tor
             x.add_(y.float(), alpha=mult)
         if bias is not None:
             x.add_(bias.float())
+        if add is not None:
+            x.add_(add)
         if w is None:
             return None
         h = R.group_rmsnorm(x, w, groups, eps, torch.float32, w_offset)
@@ -130,8 +136,10 @@ def resadd_groupnorm(x: torch.Tensor, y: Optional[torch.Tensor], w: Optional[tor
     rows, dim = x.shape
     h = (torch.empty(rows, dim, dtype=torch.float32 if out_f32 else dtype, device=x.device)
          if w is not None else None)
+    if add is not None and (add.shape != x.shape or not add.is_contiguous()):
+        raise ValueError("resadd_groupnorm: add must have the stream's shape")
     _call("dli_resadd_groupnorm", _p(x), _p(y), y.stride(0) if y is not None else 0, _p(bias),
-          float(keep), float(mult), _p(w), _p(h), dim, rows, dim, groups, float(eps), None,
+          _p(add), float(keep), float(mult), _p(w), _p(h), dim, rows, dim, groups, float(eps), None,
           float(gain), int(out_f32), float(w_offset), _dt(dtype), _st())
     return h
 
@@ -144,7 +152,7 @@ def groupnorm_rows(x: torch.Tensor, rows_idx: torch.Tensor, w: torch.Tensor, gro
         return (h * gain if gain != 1.0 else h).to(w.dtype)
     n, dim = rows_idx.shape[0], x.shape[1]
     h = torch.empty(n, dim, dtype=w.dtype, device=x.device)
-    _call("dli_resadd_groupnorm", _p(x), None, 0, None, 1.0, 1.0, _p(w), _p(h), dim, n, dim,
+    _call("dli_resadd_groupnorm", _p(x), None, 0, None, None, 1.0, 1.0, _p(w), _p(h), dim, n, dim,
           groups, float(eps), _p(rows_idx), float(gain), 0, float(w_offset), _dt(w.dtype), _st())
     return h
 
@@ -253,21 +261,23 @@ def mla_prepare(proj, cw, eps, H, d, dr, r, rot_dims, inv_freq, positions, slots
 def window_attention(q, k_cache, v_cache, dq, dv, H, G, cu_seqlens, max_seqlen, positions,
                      block_tables, block_size, window, scale, slopes=None, talk=None, gate=None,
                      chunk: int = 0, k_groups: Optional[int] = None, sink=None,
-                     head_gate: bool = False, out_scale: float = 1.0, out=None):
+                     head_gate: bool = False, out_scale: float = 1.0, out=None,
+                     keep_first: int = 0):
     """See ``reference.window_attention`` / window_attention.hip. q [T, H*dq] (storage dtype);
     caches are token-major rows; returns [T, H*dv] in the storage dtype. ``chunk`` > 0 limits
     a query to the keys of its own block of that many positions; ``k_groups`` is the number of
     key heads per cache row when it is not the number of value heads G. ``sink`` fp32 [H]
     adds exp(sink_h) to head h's softmax denominator; ``head_gate``: the gate is fp32 [T, H],
     one number per head; ``out_scale`` multiplies the output; ``out`` (rows of a wider buffer)
-    receives it."""
+    receives it. ``keep_first``: positions below it stay visible past the window."""
     Gk = G if k_groups is None else int(k_groups)
     chunk = int(chunk)
     if not q.is_cuda:
         o = R.window_attention(q, k_cache, v_cache, dq, dv, H, G, cu_seqlens, positions,
                                block_tables, block_size, window, scale, slopes, talk, gate,
                                out_dtype=q.dtype, chunk=chunk, k_groups=Gk, sink=sink,
-                               head_gate=head_gate, out_scale=out_scale)
+                               head_gate=head_gate, out_scale=out_scale,
+                               keep_first=keep_first)
         if out is not None:
             out.copy_(o)
             return out
@@ -285,7 +295,8 @@ def window_attention(q, k_cache, v_cache, dq, dv, H, G, cu_seqlens, max_seqlen, 
         rowhead = int(Gk == 1 and H > 1 and int(max_seqlen) == 1 and talk is None and gate is None
                       and slopes is None and sink is None and q.stride(0) == H * dq)
         nb = lib.dli_window_attention_mfma_workspace_bytes(S, int(max_seqlen), T, H, dv,
-                                                           int(min(window, chunk) if chunk else window),
+                                                           int(min(window, chunk) if chunk else window)
+                                                           + int(keep_first),
                                                            int(talk is not None), rowhead)
         ws = _gemm.workspace(q.device, nb) if nb else None       # key-split form (decode steps)
         rc = lib.dli_window_attention_mfma(
@@ -293,7 +304,8 @@ def window_attention(q, k_cache, v_cache, dq, dv, H, G, cu_seqlens, max_seqlen, 
             _p(out), out.stride(0), _p(gate), gate.stride(0) if gate is not None else 0,
             _p(slopes), _p(talk), _p(cu_seqlens), _p(positions), _p(block_tables),
             block_tables.stride(0), block_size, S, int(max_seqlen), H, G, dq, dv, int(window),
-            float(scale), T, _p(ws), rowhead, Gk, chunk, _p(sink), hg, float(out_scale), _st())
+            float(scale), T, _p(ws), rowhead, Gk, chunk, _p(sink), hg, float(out_scale),
+            int(keep_first), _st())
         if rc == 0:
             return out
         if rc != _NOT_SUPPORTED:
@@ -303,7 +315,7 @@ def window_attention(q, k_cache, v_cache, dq, dv, H, G, cu_seqlens, max_seqlen, 
           gate.stride(0) if gate is not None else 0, _p(slopes), _p(talk), _p(cu_seqlens),
           _p(positions), _p(block_tables), block_tables.stride(0), block_size, S,
           int(max_seqlen), H, G, dq, dv, int(window), float(scale), Gk, chunk, _p(sink), hg,
-          float(out_scale), _dt(q.dtype), _st())
+          float(out_scale), int(keep_first), _dt(q.dtype), _st())
     return out
 
 
@@ -477,27 +489,33 @@ def side_gate(gate, ids, table, col0: int) -> torch.Tensor:
 
 
 def rmsnorm_cols(src, w, eps: float, gate=None, groups: int = 1, out=None,
-                 out_scale: float = 1.0) -> torch.Tensor:
-    """RMS norm times w of the rows of an fp32 matrix that may be a column slice of a wider
-    one, times sigmoid(gate) (fp32, same shape, may be a column slice) when given, times
+                 out_scale: float = 1.0, silu_gate: bool = False, dtype=None) -> torch.Tensor:
+    """RMS norm times w (None: no weight; ``dtype`` or ``out`` then gives the storage dtype) of the rows of an fp32 matrix that may be a column slice of a wider
+    one, times sigmoid(gate) — or silu(gate) with ``silu_gate`` — (fp32, same shape, may be a
+    column slice) when given, times
     ``out_scale``; storage dtype out. With ``groups`` > 1 each row is that many equal parts,
     each normed by itself (heads). ``out`` may be a column slice of a wider buffer."""
+    dtype = w.dtype if w is not None else (out.dtype if out is not None else dtype)
     if not src.is_cuda:
         T, n = src.shape
+        if w is None:
+            w = torch.ones(n, dtype=dtype)
         o = R.rmsnorm_cols(src.reshape(T * groups, n // groups),
                            w.reshape(groups, n // groups).repeat(T, 1), eps, torch.float32,
                            gate.reshape(T * groups, n // groups) if gate is not None else None)
-        o = (o.reshape(T, n) * out_scale).to(w.dtype)
+        if silu_gate and gate is not None:
+            o = o.reshape(T, n) * gate.float()
+        o = (o.reshape(T, n) * out_scale).to(dtype)
         if out is not None:
             out.copy_(o)
             return out
         return o
     T, n = src.shape
     if out is None:
-        out = torch.empty(T, n, dtype=w.dtype, device=src.device)
+        out = torch.empty(T, n, dtype=dtype, device=src.device)
     _call("dli_rmsnorm_cols", _p(out), _p(src), src.stride(0), _p(w), T, n // groups,
           float(eps), _p(gate), gate.stride(0) if gate is not None else 0, int(groups),
-          out.stride(0), float(out_scale), _dt(w.dtype), _st())
+          out.stride(0), float(out_scale), int(silu_gate), _dt(dtype), _st())
     return out
 
 
@@ -679,4 +697,59 @@ def mlstm(proj, if_b, cap: float, norm_w, eps: float, state, mstate, slots, cu_s
         g0 = 2 * H * d + H * dv
         rmsnorm_cols(raw, norm_w, eps, gate=proj[:, g0:g0 + H * dv], groups=H, out=out,
                      out_scale=out_scale)
+    return out
+
+
+# ----------------------------------------------------------------------------- rotated designs
+def rotation_table(positions, freq) -> torch.Tensor:
+    """fp32 [T, 2 n] = cosines | sines of positions * freq (float64 [n]); the angle is formed
+    in double and rounded once."""
+    if not positions.is_cuda:
+        return R.rotation_table(positions, freq)
+    T, n = positions.shape[0], freq.shape[0]
+    out = torch.empty(T, 2 * n, dtype=torch.float32, device=positions.device)
+    _call("dli_rotation_table", _p(out), _p(positions), _p(freq), T, n, _st())
+    return out
+
+
+def rope_prepare(proj, bias, table, rot_dims: int, H, G, d, dv, kcache, vcache, slots, dtype,
+                 tied: bool):
+    """Query / cache preparation of an attention with rotated q and k
+    (``reference.rope_prepare``): bias, rotation by the step's table, k and v (or, tied, the
+    unrotated k) to the cache rows; the queries [T, H*d] come back in the storage dtype."""
+    if not proj.is_cuda:
+        return R.rope_prepare(proj, bias, table, rot_dims, H, G, d, dv, kcache, vcache, slots,
+                              dtype, tied)
+    T = proj.shape[0]
+    q = torch.empty(T, H * d, dtype=dtype, device=proj.device)
+    _call("dli_rope_prepare", _p(proj), proj.stride(0), _p(bias), _p(table), int(rot_dims), T, H,
+          G, d, dv, int(tied), _p(q), _p(kcache), _p(vcache), _p(slots), _dt(dtype), _st())
+    return q
+
+
+def retention(proj, table, rot_dims: int, decay_pow, eps: float, state, slots, cu_seqlens,
+              max_seqlen, positions, H, d, dv, dtype):
+    """Linear attention with one fixed decay per head over rotated queries and keys, per-head
+    unit-RMS read-outs, SiLU gate (``reference.retention``): [T, H*dv] in the storage dtype.
+    ``decay_pow`` fp32 [H, RETENTION_CHUNK + 1]: powers of every head's decay."""
+    if not proj.is_cuda:
+        return R.retention(proj, table, rot_dims, decay_pow[:, 1], eps, state, slots, cu_seqlens,
+                           positions, H, d, dv, dtype)
+    T = proj.shape[0]
+    S = cu_seqlens.shape[0] - 1
+    out = torch.empty(T, H * dv, dtype=dtype, device=proj.device)
+    # portions run chunk by chunk on the matrix cores, in column blocks of 64; single tokens and
+    # sizes that form does not take walk the state
+    chunked = int(max_seqlen >= 8 and d % 16 == 0 and d <= 256 and dv % 4 == 0
+                  and rot_dims % 8 == 0 and proj.stride(0) % 4 == 0)
+    cw = (64 if dv > 64 else 0) if chunked else _column_block(S, H, d, dv, max_seqlen)
+    raw = torch.empty(T, H * dv, dtype=torch.float32, device=proj.device) if cw else None
+    _call("dli_retention", _p(proj), proj.stride(0), _p(table), int(rot_dims), _p(decay_pow),
+          decay_pow.stride(0), float(d ** -0.5), float(eps), _p(state), _p(slots),
+          _p(cu_seqlens), _p(positions), _p(out), out.stride(0), S, int(max_seqlen), H, d, dv, cw,
+          _p(raw), chunked, _dt(dtype), _st())
+    if cw:                                  # no workgroup saw a whole head: norm and gate here
+        g0 = 2 * H * d + H * dv
+        rmsnorm_cols(raw, None, eps, gate=proj[:, g0:g0 + H * dv], groups=H, out=out,
+                     silu_gate=True)
     return out

@@ -469,7 +469,7 @@ def mla_prepare(proj, cw, eps, H, d, dr, r, rot_dims, inv_freq, positions, slots
 def window_attention(q, k_cache, v_cache, dq, dv, H, G, cu_seqlens, positions, block_tables,
                      block_size, window, scale, slopes=None, talk=None, gate=None,
                      out_dtype=None, chunk=0, k_groups=None, sink=None, head_gate=False,
-                     out_scale=1.0):
+                     out_scale=1.0, keep_first=0):
     """q [T, H*dq]; k_cache rows [slots, G*dq]; v_cache rows [slots, >= G*dv] (may be k_cache:
     values = the first dv columns of each kv head's... row when G == 1). Every query at position
     p attends cached positions [max(0, p-window+1), p] of its sequence. fp32 softmax; ``talk``
@@ -479,7 +479,7 @@ def window_attention(q, k_cache, v_cache, dq, dv, H, G, cu_seqlens, positions, b
     when it differs from the value heads G (1: every query head scores the whole key row).
     ``sink`` fp32 [H]: exp(sink_h) is added to head h's softmax denominator (a key without a
     value). ``head_gate``: gate is fp32 [T, H], one number per head. ``out_scale`` multiplies
-    the output."""
+    the output. ``keep_first``: the positions below it stay visible past the window."""
     T = q.shape[0]
     Gk = G if k_groups is None else k_groups
     out = torch.zeros(T, H * dv, dtype=torch.float32, device=q.device)
@@ -502,7 +502,7 @@ def window_attention(q, k_cache, v_cache, dq, dv, H, G, cu_seqlens, positions, b
         dist = (pos[:, None] - j[None, :]).float()                              # [n, ctx]
         if slopes is not None:
             sc = sc - slopes.float()[:, None, None] * dist[None]
-        vis = (dist >= 0) & (dist < window)
+        vis = (dist >= 0) & ((dist < window) | (j[None, :] < keep_first))
         if chunk:
             vis = vis & ((pos[:, None] // chunk) == (j[None, :] // chunk))
         sc = sc.masked_fill(~vis[None], float("-inf"))
@@ -967,3 +967,71 @@ def clamp_swish_mul(gu, F_, limit, out_dtype):
     g = gu[:, :F_].float().clamp(max=limit)
     u = gu[:, F_:2 * F_].float().clamp(-limit, limit)
     return (g * torch.sigmoid(1.702 * g) * (u + 1.0)).to(out_dtype)
+
+
+# ----------------------------------------------------------------------------- rotated designs
+def rotation_table(positions, freq):
+    """fp32 [T, 2 n] = cosines | sines of positions * freq (float64 [n]), rounded once."""
+    ang = positions.double()[:, None] * freq.double()[None, :]
+    return torch.cat([ang.cos(), ang.sin()], 1).float()
+
+
+def rotate_by_table(x, table, rot_dims):
+    """x [T, heads, n]: dimension i < rot_dims/2 of every head turns with i + rot_dims/2."""
+    if not rot_dims:
+        return x
+    h = rot_dims // 2
+    c, s = table[:, None, :h], table[:, None, h:]
+    u, v = x[..., :h], x[..., h:rot_dims]
+    return torch.cat([u * c - v * s, v * c + u * s, x[..., rot_dims:]], -1)
+
+
+def rope_prepare(proj, bias, table, rot_dims, H, G, d, dv, kcache, vcache, slots, out_dtype, tied):
+    """proj fp32 [T, q | k (| v)] (+ bias [that width]): q and k heads rotated by ``table``;
+    rotated k -> kcache rows; v, or with ``tied`` the unrotated k, -> vcache rows; returns q
+    [T, H*d]."""
+    T = proj.shape[0]
+    n = (H + G) * d + (0 if tied else G * dv)
+    p = proj[:, :n].float()
+    if bias is not None:
+        p = p + bias.float()
+    q = rotate_by_table(p[:, :H * d].reshape(T, H, d), table, rot_dims)
+    kraw = p[:, H * d:(H + G) * d]
+    k = rotate_by_table(kraw.reshape(T, G, d), table, rot_dims)
+    v = kraw if tied else p[:, (H + G) * d:]
+    ok = slots >= 0
+    idx = slots[ok].long()
+    kcache[idx] = k.reshape(T, G * d)[ok].to(kcache.dtype)
+    vcache[idx] = v[ok].to(vcache.dtype)
+    return q.reshape(T, H * d).to(out_dtype)
+
+
+def retention(proj, table, rot_dims, decays, eps, state, slots, cu_seqlens, positions, H, d, dv,
+              out_dtype):
+    """proj fp32 [T, 2*H*d + 2*H*dv] = [q | k | v | gate]. q and k heads rotated by ``table``, k
+    times d^(-1/2); per head S = decay_h S + k v^T, o = S^T q; every head's o divided by its
+    RMS, times silu(gate). state fp32 [slots, H, d, dv] in place; a portion whose first position
+    is 0 starts from zero; rows of sequences without a slot come out zero."""
+    T = proj.shape[0]
+    out = torch.zeros(T, H * dv, dtype=torch.float32, device=proj.device)
+    cu, sl = cu_seqlens.tolist(), slots.tolist()
+    a = decays.float().reshape(H, 1, 1)
+    p = proj.float()
+    q = rotate_by_table(p[:, :H * d].reshape(T, H, d), table, rot_dims)
+    k = rotate_by_table(p[:, H * d:2 * H * d].reshape(T, H, d), table, rot_dims) * d ** -0.5
+    v = p[:, 2 * H * d:2 * H * d + H * dv].reshape(T, H, dv)
+    g = p[:, 2 * H * d + H * dv:2 * H * (d + dv)]
+    for s in range(len(cu) - 1):
+        t0, t1 = cu[s], cu[s + 1]
+        if t1 <= t0 or sl[s] < 0:
+            continue
+        S = state[sl[s]].clone()
+        if int(positions[t0]) == 0:
+            S.zero_()
+        for t in range(t0, t1):
+            S = a * S + k[t][:, :, None] * v[t][:, None, :]
+            o = torch.einsum("hdv,hd->hv", S, q[t])
+            o = o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps)
+            out[t] = o.reshape(H * dv) * F.silu(g[t])
+        state[sl[s]] = S
+    return out.to(out_dtype)
