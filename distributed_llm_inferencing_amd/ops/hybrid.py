@@ -117,7 +117,8 @@ def resadd_groupnorm(x: torch.Tensor, y: Optional[torch.Tensor], w: Optional[tor
     the grouped RMS norm of the new x times ``w`` times ``gain`` in the storage dtype (None when
     w is None), or unrounded in fp32 with ``out_f32`` (what a token shift reads). ``w_offset``
     is added to the weight in fp32 (weights stored as offsets from one)."""
-    dtype = dtype or (w.dtype if w is not None else torch.bfloat16)
+    dtype = dtype or (w.dtype if w is not None else
+                      bias.dtype if bias is not None else torch.bfloat16)
     if not x.is_cuda:
         if keep != 1.0:
             x.mul_(keep) if keep != 0.0 else x.zero_()

@@ -157,6 +157,9 @@ def random_weights(c, seed=0):
         if L["type"] == "retention":
             dv = int(mx["vdim"])
             lin(m + "q", H * d, D), lin(m + "k", H * d, D), lin(m + "v", H * dv, D)
+            # a token's key leans towards its query: a read-out close to zero (a first token's
+            # above all) would magnify every rounding when it is divided by its RMS
+            w[m + "k"] = 0.8 * w[m + "q"] + 0.6 * w[m + "k"]
             lin(m + "g", H * dv, D, 1.5), lin(m + "o", D, H * dv)
         else:
             G = int(mx["kv_heads"])
