@@ -241,6 +241,37 @@ def run_design_lapunex(a):
                       "results": out}), flush=True)
 
 
+def run_design_bamudra(a):
+    """``--design bamudra``: prefill and decode throughput of the design at layer sizes of a
+    real model (random weights) beside a Llama of equal width, depth (= layer runs), head sizes
+    and feed-forward width, both through ``LLMEngine``. One JSON line."""
+    from dataclasses import replace
+    from distributed_llm_inferencing_amd.models.configs import LayerSpec, get_config, hybrid_config
+    D, Fw, V, Hh, G, hd = a.design_width, a.design_ff, 32000, a.design_width // 128, 8, 128
+    ff = dict(ff_kind="clamp_swish", ff=Fw, act_limit=7.0)
+    decays = tuple(1.0 - 2.0 ** (-5.0 - 6.0 * h / max(1, Hh - 1)) for h in range(Hh))
+    ret = LayerSpec("retention", heads=Hh, dim=hd, vdim=hd, decays=decays, rot_dims=hd,
+                    rot_base=10000.0, **ff)
+    att = LayerSpec("rope_attention", heads=Hh, kv_heads=G, dim=hd, vdim=hd, scale=hd ** -0.5,
+                    window=a.design_window, keep_first=4, rot_dims=64, rot_base=500000.0,
+                    bias=True, tied_values=True, **ff)
+    hyb = hybrid_config("bamudra-bench", D, V, (ret, att, ret, att), loop=(0, 2, 2),
+                        arch="bamudra", max_position=1 << 15, norm_eps=1e-5, loop_entry=False,
+                        loop_add=True)
+    runs = len(hyb.layer_runs())
+    llama = replace(get_config("llama3-8b"), name="llama-bench", hidden_size=D, num_layers=runs,
+                    num_heads=Hh, num_kv_heads=G, head_dim=hd, intermediate_size=Fw,
+                    vocab_size=V, max_position=1 << 16)
+    out = _design_sweep((hyb, llama), a, V)
+    print(json.dumps({"metric": "prefill and decode tokens/s, Bamudra design vs Llama of equal "
+                                "size (random weights)", "unit": "tokens/s", "n_gpus": 1,
+                      "dtype": "bf16", "data": "synthetic prompts, random-init weights",
+                      "config": {"width": D, "ff": Fw, "layer_runs": runs, "heads": Hh,
+                                 "kv_heads": G, "head_dim": hd, "window": a.design_window,
+                                 "keep_first": 4, "retention_heads": Hh},
+                      "results": out}), flush=True)
+
+
 def run_design(a):
     """``--design buborax``: prefill and decode throughput of the hybrid design at layer sizes
     of a real model (random weights), beside a Llama of equal width, depth (= layer runs),
@@ -465,11 +496,12 @@ def main():
                     help="N>1: pp = layer-sharded pipeline (dense, default), ep = expert "
                          "parallel (MoE), tp = tensor-parallel ablation, dp = independent "
                          "replicas")
-    ap.add_argument("--design", default=None, choices=["buborax", "pulunex", "risutar", "lapunex"],
+    ap.add_argument("--design", default=None, choices=["buborax", "pulunex", "risutar", "lapunex", "bamudra"],
                     help="instead of the headline workload: prefill / decode throughput of "
                          "this design at real layer sizes beside the closest model of equal "
-                         "size (buborax: Llama, pulunex, risutar and lapunex: Mixtral)")
-    ap.add_argument("--design-models", default="buborax,llama,pulunex,mixtral,risutar,lapunex",
+                         "size (buborax and bamudra: Llama, pulunex, risutar and lapunex: "
+                         "Mixtral)")
+    ap.add_argument("--design-models", default="buborax,llama,pulunex,mixtral,risutar,lapunex,bamudra",
                     help="which of the design and its comparison model to run")
     ap.add_argument("--design-width", type=int, default=4096)
     ap.add_argument("--design-ff", type=int, default=14336)
@@ -485,6 +517,8 @@ def main():
             return run_design_risutar(a)
         if a.design == "lapunex":
             return run_design_lapunex(a)
+        if a.design == "bamudra":
+            return run_design_bamudra(a)
         return run_design_pulunex(a) if a.design == "pulunex" else run_design(a)
 
     from distributed_llm_inferencing_amd import launch

@@ -106,7 +106,9 @@ _SIGS = {
     "dli_sink_prepare": [P, I, P, P, F, I, I, I, I, I, I, P, F, P, P, P, P, P, I, P],
     "dli_scalar_recurrence": [P, I, I, P, P, F, P, F, P, P, P, P, P, P, I, F, I, I, I, I, I,
                               I, P, I, P],
-    # rotated designs (rotary.hip, retention.hip)
+    # rotated designs (rotary.hip, retention.hip, swa_attention.hip)
+    "dli_swa_attention": [P, I, P, L, P, L, P, I, P, P, P, I, I, I, I, I, I, I, I, I, F, P, P],
+    "dli_swa_attention_workspace_bytes": [I, I, I, I, I, I, I],
     "dli_rotation_table": [P, P, P, I, I, P],
     "dli_rope_prepare": [P, I, P, P, I, I, I, I, I, I, I, P, P, P, P, I, P],
     "dli_retention": [P, I, P, I, P, I, F, F, P, P, P, P, P, I, I, I, I, I, I, I, P, I, I, P],

@@ -289,8 +289,23 @@ def window_attention(q, k_cache, v_cache, dq, dv, H, G, cu_seqlens, max_seqlen, 
         out = torch.empty(T, H * dv, dtype=q.dtype, device=q.device)
     hg = int(bool(head_gate))
     if q.dtype == torch.bfloat16 and MFMA_ATTENTION:
-        # the MFMA form; shapes it does not take (odd head sizes, > 32 heads) fall through
         lib = N.require_native()
+        if (dq == dv and Gk == G and not chunk and slopes is None and talk is None and gate is None
+                and sink is None and out_scale == 1.0):
+            # plain grouped-query attention: the dedicated kernels (head sizes 64 and 128)
+            nb = lib.dli_swa_attention_workspace_bytes(S, int(max_seqlen), H, G, dq, int(window),
+                                                       int(keep_first))
+            ws = _gemm.workspace(q.device, nb) if nb else None
+            rc = lib.dli_swa_attention(
+                _p(q), q.stride(0), _p(k_cache), k_cache.stride(0), _p(v_cache),
+                v_cache.stride(0), _p(out), out.stride(0), _p(cu_seqlens), _p(positions),
+                _p(block_tables), block_tables.stride(0), block_size, S, int(max_seqlen), H, G, dq,
+                int(window), int(keep_first), float(scale), _p(ws), _st())
+            if rc == 0:
+                return out
+            if rc != _NOT_SUPPORTED:
+                raise RuntimeError(f"dli_swa_attention failed with hipError {rc}")
+        # the MFMA form; shapes it does not take (odd head sizes, > 32 heads) fall through
         # decode steps of heads that share one cached row per position (latent attention):
         # the heads become the query rows of a one-head problem
         rowhead = int(Gk == 1 and H > 1 and int(max_seqlen) == 1 and talk is None and gate is None
