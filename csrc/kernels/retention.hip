@@ -18,8 +18,11 @@
 // padded by 8 floats, which spreads every 16-lane group over all banks.
 //
 // With more than one column block no workgroup sees a whole head: o_t leaves in fp32 (`raw`)
-// and the caller norms and gates it. Single tokens (decode steps) and shapes this form does
-// not take run the walk of recurrent_scalar.hip.
+// and the caller norms and gates it.
+//
+// Decode steps (one token a sequence) stream the state through registers, with rotation, norm
+// and gate in the same launch. Shapes neither form takes, and portions of a few tokens, run the
+// walk of recurrent_scalar.hip.
 #include "common.h"
 
 // recurrent_scalar.hip
@@ -30,15 +33,16 @@ int retention_walk(const float* proj, int ldp, const float* table, int rot, cons
 
 namespace {
 
-template <typename S> __device__ __forceinline__ void stf4(S* p, f32x4 v);
-template <> __device__ __forceinline__ void stf4<float>(float* p, f32x4 v) {
-  *reinterpret_cast<f32x4*>(p) = v;
-}
-template <> __device__ __forceinline__ void stf4<u16>(u16* p, f32x4 v) {
-  uint2 pk;
-  pk.x = pack2bf(v[0], v[1]);
-  pk.y = pack2bf(v[2], v[3]);
-  *reinterpret_cast<uint2*>(p) = pk;
+// four elements at index i of the output, bf16 (dt 0) or fp32 (dt 1)
+__device__ __forceinline__ void store4(void* out, int dt, long i, f32x4 v) {
+  if (dt == 0) {
+    uint2 pk;
+    pk.x = pack2bf(v[0], v[1]);
+    pk.y = pack2bf(v[2], v[3]);
+    *reinterpret_cast<uint2*>((u16*)out + i) = pk;
+  } else {
+    *reinterpret_cast<f32x4*>((float*)out + i) = v;
+  }
 }
 
 constexpr int CW = 64;            // state columns of a workgroup
@@ -54,14 +58,15 @@ struct RetentionArgs {
   const int* slots; const int* cu; const int* positions;
   void* out; int ldo;              // [T, H*dv]
   float* raw;                      // several column blocks: o_t, fp32 [T, H*dv]
-  int H, d, dv;
+  int H, d, dv, dt;
 };
 
-// C tokens a chunk; NT: 16-row state tiles a wave accumulates (d <= 32 NT)
-template <typename S, int C, int NT>
+// C tokens a chunk; NT: 16-row state tiles a wave accumulates (d <= 32 NT); D: d when it is known
+// at compile time (else 0)
+template <int C, int NT, int D>
 __global__ void __launch_bounds__(NTH) retention_chunk_kernel(RetentionArgs a) {
   extern __shared__ __attribute__((aligned(16))) float sm[];
-  const int d = a.d, dv = a.dv, H = a.H;
+  const int d = D ? D : a.d, dv = a.dv, H = a.H;
   const int ldq = d + PAD;
   constexpr int ldc = C + PAD;
   float* Qs = sm;                          // [C][ldq] rotated queries
@@ -82,7 +87,7 @@ __global__ void __launch_bounds__(NTH) retention_chunk_kernel(RetentionArgs a) {
       const long o = (long)(t0 + i / ncol);
       const int c = h * dv + c0 + i % ncol;
       if (a.raw != nullptr) a.raw[o * H * dv + c] = 0.f;
-      else if (sizeof(S) == 2) ((u16*)a.out)[o * a.ldo + c] = 0;
+      else if (a.dt == 0) ((u16*)a.out)[o * a.ldo + c] = 0;
       else ((float*)a.out)[o * a.ldo + c] = 0.f;
     }
     return;
@@ -106,9 +111,10 @@ __global__ void __launch_bounds__(NTH) retention_chunk_kernel(RetentionArgs a) {
       *reinterpret_cast<f32x4*>(St + (ct * 16 + fr) * ldq + dt * 16 + 4 * q) = sacc[n];
     }
   }
-  // staging: a unit is a pair of rotated quads (c, c + rot/2) or one quad that passes
-  const int hr = a.rot >> 1, rq = hr >> 2, up = rq + ((d - a.rot) >> 2);
-  constexpr int MAXU = (C * NT * 8 + NTH - 1) / NTH;
+  // staging: a unit is two quads of a row, rotated partners (c, c + rot/2) or, past the rotated
+  // dims, neighbours: d/8 units a row whatever rotates
+  const int hr = a.rot >> 1, rq = hr >> 2, up = d >> 3;
+  constexpr int MAXU = (C * NT * 4 + NTH - 1) / NTH;
   constexpr int VU = C * (CW / 4) / NTH;
   f32x4 pq[MAXU][2], pk[MAXU][2], tb[MAXU][2], pv[VU];
   const int voff = 2 * H * d + h * dv + c0;
@@ -120,13 +126,13 @@ __global__ void __launch_bounds__(NTH) retention_chunk_kernel(RetentionArgs a) {
       const int r = it / up, k = it - r * up;
       if (r < n) {
         const bool pair = k < rq;
-        const int c = pair ? 4 * k : a.rot + 4 * (k - rq);
-        const float* p = a.proj + (long)(tc + r) * a.ldp + h * d + c;
-        pq[u][0] = *reinterpret_cast<const f32x4*>(p);
-        pk[u][0] = *reinterpret_cast<const f32x4*>(p + H * d);
+        const int c = pair ? 4 * k : a.rot + 8 * (k - rq), c2 = pair ? c + hr : c + 4;
+        const float* p = a.proj + (long)(tc + r) * a.ldp + h * d;
+        pq[u][0] = *reinterpret_cast<const f32x4*>(p + c);
+        pq[u][1] = *reinterpret_cast<const f32x4*>(p + c2);
+        pk[u][0] = *reinterpret_cast<const f32x4*>(p + H * d + c);
+        pk[u][1] = *reinterpret_cast<const f32x4*>(p + H * d + c2);
         if (pair) {
-          pq[u][1] = *reinterpret_cast<const f32x4*>(p + hr);
-          pk[u][1] = *reinterpret_cast<const f32x4*>(p + H * d + hr);
           const float* tp = a.table + (long)(tc + r) * a.rot + c;
           tb[u][0] = *reinterpret_cast<const f32x4*>(tp);
           tb[u][1] = *reinterpret_cast<const f32x4*>(tp + hr);
@@ -152,26 +158,25 @@ __global__ void __launch_bounds__(NTH) retention_chunk_kernel(RetentionArgs a) {
       const int r = it / up, k = it - r * up;
       if (r >= rows) continue;
       const bool pair = k < rq;
-      const int c = pair ? 4 * k : a.rot + 4 * (k - rq);
-      float* qd = Qs + r * ldq + c;
-      float* kd = Ks + r * ldq + c;
-      if (r >= n) {
-        *reinterpret_cast<f32x4*>(qd) = zero;
-        *reinterpret_cast<f32x4*>(kd) = zero;
+      const int c = pair ? 4 * k : a.rot + 8 * (k - rq), c2 = pair ? c + hr : c + 4;
+      f32x4 q0 = zero, q1 = zero, k0 = zero, k1 = zero;
+      if (r < n) {
+        q0 = pq[u][0]; q1 = pq[u][1];
+        k0 = pk[u][0]; k1 = pk[u][1];
         if (pair) {
-          *reinterpret_cast<f32x4*>(qd + hr) = zero;
-          *reinterpret_cast<f32x4*>(kd + hr) = zero;
+          const f32x4 cs = tb[u][0], sn = tb[u][1];
+          q0 = pq[u][0] * cs - pq[u][1] * sn;
+          q1 = pq[u][1] * cs + pq[u][0] * sn;
+          k0 = pk[u][0] * cs - pk[u][1] * sn;
+          k1 = pk[u][1] * cs + pk[u][0] * sn;
         }
-      } else if (pair) {
-        const f32x4 cs = tb[u][0], sn = tb[u][1];
-        *reinterpret_cast<f32x4*>(qd) = pq[u][0] * cs - pq[u][1] * sn;
-        *reinterpret_cast<f32x4*>(qd + hr) = pq[u][1] * cs + pq[u][0] * sn;
-        *reinterpret_cast<f32x4*>(kd) = (pk[u][0] * cs - pk[u][1] * sn) * a.kscale;
-        *reinterpret_cast<f32x4*>(kd + hr) = (pk[u][1] * cs + pk[u][0] * sn) * a.kscale;
-      } else {
-        *reinterpret_cast<f32x4*>(qd) = pq[u][0];
-        *reinterpret_cast<f32x4*>(kd) = pk[u][0] * a.kscale;
+        k0 *= a.kscale;
+        k1 *= a.kscale;
       }
+      *reinterpret_cast<f32x4*>(Qs + r * ldq + c) = q0;
+      *reinterpret_cast<f32x4*>(Qs + r * ldq + c2) = q1;
+      *reinterpret_cast<f32x4*>(Ks + r * ldq + c) = k0;
+      *reinterpret_cast<f32x4*>(Ks + r * ldq + c2) = k1;
     }
 #pragma unroll
     for (int u = 0; u < VU; ++u) {
@@ -196,6 +201,7 @@ __global__ void __launch_bounds__(NTH) retention_chunk_kernel(RetentionArgs a) {
       const float* kp = Ks + (jt * 16 + fr) * ldq + 4 * q;
       const float* qp = Qs + (it * 16 + fr) * ldq + 4 * q;
       f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll (D ? 4 : 1)
       for (int x = 0; x < d; x += 16) {
         const f32x4 kf = *reinterpret_cast<const f32x4*>(kp + x);
         const f32x4 qf = *reinterpret_cast<const f32x4*>(qp + x);
@@ -212,20 +218,28 @@ __global__ void __launch_bounds__(NTH) retention_chunk_kernel(RetentionArgs a) {
     // this wave's column tile for tokens of row tiles dt0 and (chunk of four) 3 - dt0
     f32x4 oacc[C / 32];
 #pragma unroll
-    for (int m = 0; m < C / 32; ++m) {
-      const int it = m == 0 ? dt0 : 3 - dt0;
-      oacc[m] = f32x4{0.f, 0.f, 0.f, 0.f};
-      if (it >= nt) continue;
+    for (int m = 0; m < C / 32; ++m) oacc[m] = f32x4{0.f, 0.f, 0.f, 0.f};
+    {
       const float* vp = St + (ct * 16 + fr) * ldq + 4 * q;
-      const float* qp = Qs + (it * 16 + fr) * ldq + 4 * q;
+      const float* qp = Qs + fr * ldq + 4 * q;
+#pragma unroll (D ? 4 : 1)
       for (int x = 0; x < d; x += 16) {
         const f32x4 sf = *reinterpret_cast<const f32x4*>(vp + x);
-        const f32x4 qf = *reinterpret_cast<const f32x4*>(qp + x);
 #pragma unroll
-        for (int i = 0; i < 4; ++i)
-          oacc[m] = __builtin_amdgcn_mfma_f32_16x16x4f32(sf[i], qf[i], oacc[m], 0, 0, 0);
+        for (int m = 0; m < C / 32; ++m) {
+          const int it = m == 0 ? dt0 : 3 - dt0;
+          if (it >= nt) continue;
+          const f32x4 qf = *reinterpret_cast<const f32x4*>(qp + it * 16 * ldq + x);
+#pragma unroll
+          for (int i = 0; i < 4; ++i)
+            oacc[m] = __builtin_amdgcn_mfma_f32_16x16x4f32(sf[i], qf[i], oacc[m], 0, 0, 0);
+        }
       }
-      oacc[m] *= pw[it * 16 + fr + 1];
+#pragma unroll
+      for (int m = 0; m < C / 32; ++m) {
+        const int it = m == 0 ? dt0 : 3 - dt0;
+        if (it < nt) oacc[m] *= pw[it * 16 + fr + 1];
+      }
     }
     // ---- the state after the chunk: key columns (dims) x decayed values
     f32x4 vf[C / 16];
@@ -300,7 +314,7 @@ __global__ void __launch_bounds__(NTH) retention_chunk_kernel(RetentionArgs a) {
         f32x4 o;
 #pragma unroll
         for (int i = 0; i < 4; ++i) o[i] = oacc[m][i] * rs * (g[i] / (1.f + expf(-g[i])));
-        stf4((S*)a.out + t * a.ldo + h * dv + c0 + c, o);
+        store4(a.out, a.dt, t * a.ldo + h * dv + c0 + c, o);
       }
     }
   }
@@ -314,27 +328,124 @@ __global__ void __launch_bounds__(NTH) retention_chunk_kernel(RetentionArgs a) {
   }
 }
 
-template <typename S, int C, int NT>
+template <int C, int NT, int D>
 int launch_chunks(const RetentionArgs& a, int num_seqs, hipStream_t st) {
   const size_t sh = ((size_t)2 * C * (a.d + PAD) + (size_t)(CW + C) * (C + PAD) +
                      (size_t)CW * (a.d + PAD) + C + 4 + C * 4) * 4;
   if (sh > 160 * 1024) return (int)hipErrorInvalidValue;
   if (sh > 48 * 1024) {
-    hipError_t e = hipFuncSetAttribute((const void*)retention_chunk_kernel<S, C, NT>,
+    hipError_t e = hipFuncSetAttribute((const void*)retention_chunk_kernel<C, NT, D>,
                                        hipFuncAttributeMaxDynamicSharedMemorySize, (int)sh);
     if (e != hipSuccess) return (int)e;
   }
   dim3 grid(a.H, num_seqs, (a.dv + CW - 1) / CW);
-  retention_chunk_kernel<S, C, NT><<<grid, NTH, sh, st>>>(a);
+  retention_chunk_kernel<C, NT, D><<<grid, NTH, sh, st>>>(a);
   DLI_RETURN_LAUNCH();
 }
 
-template <typename S>
 int launch_chunks_any(const RetentionArgs& a, int num_seqs, hipStream_t st) {
-  if (a.d <= 32) return launch_chunks<S, 64, 1>(a, num_seqs, st);
-  if (a.d <= 64) return launch_chunks<S, 64, 2>(a, num_seqs, st);
-  if (a.d <= 128) return launch_chunks<S, 64, 4>(a, num_seqs, st);
-  return launch_chunks<S, 32, 8>(a, num_seqs, st);
+  if (a.d == 64) return launch_chunks<64, 2, 64>(a, num_seqs, st);
+  if (a.d == 128) return launch_chunks<64, 4, 128>(a, num_seqs, st);
+  if (a.d == 256) return launch_chunks<32, 8, 256>(a, num_seqs, st);
+  if (a.d <= 32) return launch_chunks<64, 1, 0>(a, num_seqs, st);
+  if (a.d <= 64) return launch_chunks<64, 2, 0>(a, num_seqs, st);
+  if (a.d <= 128) return launch_chunks<64, 4, 0>(a, num_seqs, st);
+  return launch_chunks<32, 8, 0>(a, num_seqs, st);
+}
+
+// One token a sequence (decode steps): a workgroup per (head, sequence). Thread = (column quad
+// cq of QP, row group rg of RG = 256 / QP); its R = ceil(d / RG) state quads stream through
+// registers, all in flight at once: one read and one write per element.
+template <int R>
+__global__ void __launch_bounds__(256, R >= 32 ? 2 : 4) retention_step_kernel(RetentionArgs a, int qp_log2) {
+  extern __shared__ __attribute__((aligned(16))) float sm[];
+  const int d = a.d, dv = a.dv, H = a.H;
+  const int QP = 1 << qp_log2, RG = 256 >> qp_log2;
+  float* qs = sm;                          // [d], padded to a multiple of 4
+  float* ks = qs + ((d + 3) & ~3);         // [d]
+  float* ov = ks + ((d + 3) & ~3);         // [RG][4 QP] partial read-outs
+  float* red = ov + RG * 4 * QP;           // [16]
+  const int h = blockIdx.x, s = blockIdx.y;
+  const int t = a.cu[s];
+  if (a.cu[s + 1] <= t) return;
+  const int tid = threadIdx.x, cq = tid & (QP - 1), rg = tid >> qp_log2;
+  const int slot = a.slots[s];
+  const long oi = (long)t * a.ldo + h * dv;
+  const bool col = 4 * cq < dv;
+  if (slot < 0) {                          // padding rows of a captured step
+    if (col && rg == 0) store4(a.out, a.dt, oi + 4 * cq, f32x4{0.f, 0.f, 0.f, 0.f});
+    return;
+  }
+  const bool fresh = a.positions[t] == 0;
+  float* sp = a.state + ((long)slot * H + h) * d * dv + 4 * cq;
+  f32x4 S[R];
+#pragma unroll
+  for (int i = 0; i < R; ++i) {
+    const int r = rg + i * RG;
+    S[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (!fresh && col && r < d) S[i] = *reinterpret_cast<const f32x4*>(sp + (long)r * dv);
+  }
+  const float* row = a.proj + (long)t * a.ldp;
+  f32x4 v = {0.f, 0.f, 0.f, 0.f};
+  if (col) v = *reinterpret_cast<const f32x4*>(row + 2 * H * d + h * dv + 4 * cq);
+  const int hr = a.rot >> 1;
+  for (int i = tid; i < d; i += 256) {
+    float q = row[h * d + i], k = row[H * d + h * d + i];
+    if (i < a.rot) {
+      const bool second = i >= hr;
+      const int ci = second ? i - hr : i, pi = second ? i - hr : i + hr;
+      const float* tb = a.table + (long)t * a.rot;
+      const float cs = tb[ci], sn = second ? tb[hr + ci] : -tb[hr + ci];
+      q = q * cs + row[h * d + pi] * sn;
+      k = k * cs + row[H * d + h * d + pi] * sn;
+    }
+    qs[i] = q;
+    ks[i] = k * a.kscale;
+  }
+  const float dec = a.pw[(long)h * a.ldw + 1];
+  __syncthreads();
+  f32x4 o = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int i = 0; i < R; ++i) {
+    const int r = rg + i * RG;
+    if (r < d) {
+      S[i] = dec * S[i] + ks[r] * v;
+      o += qs[r] * S[i];
+      if (col) *reinterpret_cast<f32x4*>(sp + (long)r * dv) = S[i];
+    }
+  }
+  *reinterpret_cast<f32x4*>(ov + (rg * QP + cq) * 4) = o;
+  __syncthreads();
+  float ss = 0.f;
+  o = f32x4{0.f, 0.f, 0.f, 0.f};
+  if (rg == 0) {
+    for (int g = 0; g < RG; ++g) o += *reinterpret_cast<const f32x4*>(ov + (g * QP + cq) * 4);
+    ss = (o[0] * o[0] + o[1] * o[1]) + (o[2] * o[2] + o[3] * o[3]);
+  }
+  ss = block_sum(ss, red);
+  if (rg == 0 && col) {
+    const float rs = 1.f / sqrtf(ss / (float)dv + a.eps);
+    const f32x4 g = *reinterpret_cast<const f32x4*>(row + 2 * H * d + H * dv + h * dv + 4 * cq);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) o[i] *= rs * (g[i] / (1.f + expf(-g[i])));
+    store4(a.out, a.dt, oi + 4 * cq, o);
+  }
+}
+
+int launch_step(const RetentionArgs& a, int num_seqs, hipStream_t st) {
+  int lg = 0;
+  while ((4 << lg) < a.dv) ++lg;           // column quads, rounded up to a power of two
+  if (lg > 8) return (int)hipErrorNotSupported;
+  const int RG = 256 >> lg, R = (a.d + RG - 1) / RG;
+  const size_t sh = ((size_t)2 * ((a.d + 3) & ~3) + 1024 + 16) * 4;
+  if (R > 32 || sh > 48 * 1024) return (int)hipErrorNotSupported;
+  dim3 grid(a.H, num_seqs);
+  if (R <= 1) retention_step_kernel<1><<<grid, 256, sh, st>>>(a, lg);
+  else if (R <= 4) retention_step_kernel<4><<<grid, 256, sh, st>>>(a, lg);
+  else if (R <= 8) retention_step_kernel<8><<<grid, 256, sh, st>>>(a, lg);
+  else if (R <= 16) retention_step_kernel<16><<<grid, 256, sh, st>>>(a, lg);
+  else retention_step_kernel<32><<<grid, 256, sh, st>>>(a, lg);
+  DLI_RETURN_LAUNCH();
 }
 
 }  // namespace
@@ -353,17 +464,23 @@ extern "C" int dli_retention(const float* proj, int ldp, const float* table, int
       slots == nullptr || decay_pow == nullptr || out == nullptr || (dt != 0 && dt != 1) ||
       num_seqs > 65535)
     return (int)hipErrorInvalidValue;
+  const uintptr_t mis = (uintptr_t)proj | (uintptr_t)table | (uintptr_t)out | (uintptr_t)raw |
+                        (uintptr_t)state;
+  const bool quads = dv % 4 == 0 && ldp % 4 == 0 && ldo % 4 == 0 && (H * d) % 2 == 0 &&
+                     mis % 16 == 0;
+  RetentionArgs a{proj, ldp, table, rot, decay_pow, ldd, kscale, eps, state, slots, cu,
+                  positions, out, ldo, raw, H, d, dv, dt};
   if (!chunked) {
+    if (max_seqlen == 1 && quads && raw == nullptr) {
+      const int rc = launch_step(a, num_seqs, st);
+      if (rc != (int)hipErrorNotSupported) return rc;
+    }
     if (cw == 0 || cw >= dv) cw = dv;
     if ((cw < dv) != (raw != nullptr)) return (int)hipErrorInvalidValue;
     return retention_walk(proj, ldp, table, rot, decay_pow, ldd, eps, state, slots, cu, positions,
                           out, ldo, num_seqs, H, d, dv, cw, raw, dt, st);
   }
-  const uintptr_t mis = (uintptr_t)proj | (uintptr_t)table | (uintptr_t)out | (uintptr_t)raw;
-  if (d % 16 || d > 256 || dv % 4 || rot % 8 || ldp % 4 || ldo % 4 || mis % 16 ||
-      (dv > CW) != (raw != nullptr))
+  if (d % 16 || d > 256 || !quads || rot % 8 || (dv > CW) != (raw != nullptr))
     return (int)hipErrorInvalidValue;
-  RetentionArgs a{proj, ldp, table, rot, decay_pow, ldd, kscale, eps, state, slots, cu,
-                  positions, out, ldo, raw, H, d, dv};
-  return dt == 0 ? launch_chunks_any<u16>(a, num_seqs, st) : launch_chunks_any<float>(a, num_seqs, st);
+  return launch_chunks_any(a, num_seqs, st);
 }

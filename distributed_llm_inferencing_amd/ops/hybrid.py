@@ -758,7 +758,13 @@ def retention(proj, table, rot_dims: int, decay_pow, eps: float, state, slots, c
     # sizes that form does not take walk the state
     chunked = int(max_seqlen >= 8 and d % 16 == 0 and d <= 256 and dv % 4 == 0
                   and rot_dims % 8 == 0 and proj.stride(0) % 4 == 0)
-    cw = (64 if dv > 64 else 0) if chunked else _column_block(S, H, d, dv, max_seqlen)
+    quads = 1 << max(0, (dv + 3) // 4 - 1).bit_length()           # of a row, as a power of two
+    if chunked:
+        cw = 64 if dv > 64 else 0
+    elif int(max_seqlen) == 1 and dv % 4 == 0 and H * d % 2 == 0 and quads <= 256 and d * quads <= 8192:
+        cw = 0                              # decode rows: a head's state streams through one workgroup
+    else:
+        cw = _column_block(S, H, d, dv, max_seqlen)
     raw = torch.empty(T, H * dv, dtype=torch.float32, device=proj.device) if cw else None
     _call("dli_retention", _p(proj), proj.stride(0), _p(table), int(rot_dims), _p(decay_pow),
           decay_pow.stride(0), float(d ** -0.5), float(eps), _p(state), _p(slots),
