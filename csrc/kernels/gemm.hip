@@ -80,7 +80,8 @@ extern "C" int dli_gemm(const void* A, int lda, const void* W, int ldw, void* C,
   if (M <= 0 || N <= 0) return 0;
   if (((tile_cfg < 29 || tile_cfg > 33) && K % BK) || lda % 8 || ldw % 8 || splits < 1)
     return (int)hipErrorInvalidValue;
-  if (epi == EPI_SILU && N % 32) return (int)hipErrorInvalidValue;
+  if (epi_pairs(epi) && N % 32) return (int)hipErrorInvalidValue;
+  if (epi == EPI_CLAMP && (bias == nullptr || group_off != nullptr)) return (int)hipErrorInvalidValue;
   if (splits > 1 && ws == nullptr) return (int)hipErrorInvalidValue;
   if (groups < 1) groups = 1;
   const int* go = group_off;

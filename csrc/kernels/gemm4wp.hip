@@ -216,7 +216,7 @@ __global__ void __launch_bounds__(256, 1) gemm4wp_kernel(
           const f32x4 g = vget(acc[i][j]), u = vget(acc[i][j + 1]);
           const int gcol = wc0 + 16 * j;
           if (row < M && gcol < N)
-            store_silu_quad(C, ldc, row, (gcol >> 5) * 16 + 4 * fq, g, u, vec);
+            store_pair_quad(C, ldc, row, (gcol >> 5) * 16 + 4 * fq, g, u, vec);
         }
       }
     } else {

@@ -294,7 +294,8 @@ __global__ void __launch_bounds__(512) gemm8p_kernel(
     return;
   }
   const bool vec = out_vec<EPI>(C, ldc, N, bias);
-  if (EPI == EPI_SILU) {
+  if (epi_pairs(EPI)) {
+    const float lim = pair_const<EPI>(bias);
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
       const int row = wr0 + 16 * i + fr;
@@ -303,8 +304,8 @@ __global__ void __launch_bounds__(512) gemm8p_kernel(
       for (int j = 0; j < 4; j += 2) {
         const int gcol = wc0 + 16 * j;
         if (gcol < N)
-          store_silu_quad(C, ldc, row0 + row, (gcol >> 5) * 16 + 4 * fq, acc[i][j],
-                          acc[i][j + 1], vec);
+          store_pair_quad<EPI>(C, ldc, row0 + row, (gcol >> 5) * 16 + 4 * fq, acc[i][j],
+                          acc[i][j + 1], vec, lim);
       }
     }
     return;
@@ -531,7 +532,8 @@ __global__ void __launch_bounds__(512) gemm8p224_kernel(
     return;
   }
   const bool vec = out_vec<EPI>(C, ldc, N, bias);
-  if (EPI == EPI_SILU) {
+  if (epi_pairs(EPI)) {
+    const float lim = pair_const<EPI>(bias);
     // block 6 of wave wn = 0 (gate) pairs with block 0 of wave wn = 1 (up): through LDS
     __syncthreads();                               // every wave is past its last LDS read
     float* xch = reinterpret_cast<float*>(smem) + (2 * g + wm) * 1024;   // 64 x 16 fp32
@@ -552,21 +554,21 @@ __global__ void __launch_bounds__(512) gemm8p224_kernel(
         for (int q = 0; q < 3; ++q) {
           const int gcol = wc0 + 32 * q;
           if (gcol < N)
-            store_silu_quad(C, ldc, row0 + row, (gcol >> 5) * 16 + 4 * fq, acc[i][2 * q],
-                            acc[i][2 * q + 1], vec);
+            store_pair_quad<EPI>(C, ldc, row0 + row, (gcol >> 5) * 16 + 4 * fq, acc[i][2 * q],
+                            acc[i][2 * q + 1], vec, lim);
         }
         const int gcol = wc0 + 16 * 6;
         if (gcol < N) {
           const f32x4 up = *reinterpret_cast<const f32x4*>(xch + (16 * i + fr) * 16 + 4 * fq);
-          store_silu_quad(C, ldc, row0 + row, (gcol >> 5) * 16 + 4 * fq, acc[i][6], up, vec);
+          store_pair_quad<EPI>(C, ldc, row0 + row, (gcol >> 5) * 16 + 4 * fq, acc[i][6], up, vec, lim);
         }
       } else {
 #pragma unroll
         for (int q = 0; q < 3; ++q) {
           const int gcol = wc0 + 16 + 32 * q;
           if (gcol < N)
-            store_silu_quad(C, ldc, row0 + row, (gcol >> 5) * 16 + 4 * fq, acc[i][2 * q + 1],
-                            acc[i][2 * q + 2], vec);
+            store_pair_quad<EPI>(C, ldc, row0 + row, (gcol >> 5) * 16 + 4 * fq, acc[i][2 * q + 1],
+                            acc[i][2 * q + 2], vec, lim);
         }
       }
     }
@@ -779,7 +781,8 @@ __global__ void __launch_bounds__(512) gemm8p128_kernel(
     return;
   }
   const bool vec = out_vec<EPI>(C, ldc, N, bias);
-  if (EPI == EPI_SILU) {
+  if (epi_pairs(EPI)) {
+    const float lim = pair_const<EPI>(bias);
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int row = wr0 + 16 * i + fr;
@@ -788,8 +791,8 @@ __global__ void __launch_bounds__(512) gemm8p128_kernel(
       for (int q = 0; q < 2; ++q) {
         const int gcol = wc0 + 32 * q;
         if (gcol < N)
-          store_silu_quad(C, ldc, row0 + row, (gcol >> 5) * 16 + 4 * fq, acc[i][2 * q],
-                          acc[i][2 * q + 1], vec);
+          store_pair_quad<EPI>(C, ldc, row0 + row, (gcol >> 5) * 16 + 4 * fq, acc[i][2 * q],
+                          acc[i][2 * q + 1], vec, lim);
       }
     }
     return;
@@ -823,7 +826,7 @@ template <int EPI, int VAR = 0>
 static int launch_8p(const void* A, int lda, const void* W, int ldw, void* C, int ldc, int M,
                      int N, int K, int splits, const void* bias, void* ws, const int* group_off,
                      int groups, hipStream_t st) {
-  if (EPI == EPI_SILU && N % 64) return (int)hipErrorInvalidValue;
+  if (epi_pairs(EPI) && N % 64) return (int)hipErrorInvalidValue;
   const int tiles = ((M + 255) / 256) * ((N + 255) / 256);
   int ksl = K / splits;
   ksl = (ksl / BK) * BK;
@@ -839,7 +842,7 @@ static int launch_8p(const void* A, int lda, const void* W, int ldw, void* C, in
   gemm8p_kernel<EPI, VAR><<<grid, 512, lds, st>>>((const u16*)A, lda, (const u16*)W, ldw, C, ldc, M,
                                              N, K, ksl, (const u16*)bias, (float*)ws, group_off);
   if (splits > 1 && C != nullptr) {
-    const int outN = (EPI == EPI_SILU) ? N / 2 : N;
+    const int outN = epi_pairs(EPI) ? N / 2 : N;
     const long total = (long)M * outN;
     splitk_reduce_kernel<EPI><<<(int)((total + 255) / 256), 256, 0, st>>>(
         C, ldc, (const float*)ws, M, N, splits, (const u16*)bias);
@@ -851,7 +854,7 @@ template <int EPI>
 static int launch_8p224(const void* A, int lda, const void* W, int ldw, void* C, int ldc,
                         int M, int N, int K, int splits, const void* bias, void* ws,
                         const int* group_off, int groups, hipStream_t st) {
-  if (EPI == EPI_SILU && N % 32) return (int)hipErrorInvalidValue;
+  if (epi_pairs(EPI) && N % 32) return (int)hipErrorInvalidValue;
   const int tiles = ((M + 255) / 256) * ((N + 223) / 224);
   int ksl = K / splits;
   ksl = (ksl / BK) * BK;
@@ -868,7 +871,7 @@ static int launch_8p224(const void* A, int lda, const void* W, int ldw, void* C,
                                                 M, N, K, ksl, (const u16*)bias, (float*)ws,
                                                 group_off);
   if (splits > 1 && C != nullptr) {
-    const int outN = (EPI == EPI_SILU) ? N / 2 : N;
+    const int outN = epi_pairs(EPI) ? N / 2 : N;
     const long total = (long)M * outN;
     splitk_reduce_kernel<EPI><<<(int)((total + 255) / 256), 256, 0, st>>>(
         C, ldc, (const float*)ws, M, N, splits, (const u16*)bias);
@@ -880,7 +883,7 @@ template <int EPI>
 static int launch_8p128(const void* A, int lda, const void* W, int ldw, void* C, int ldc,
                         int M, int N, int K, int splits, const void* bias, void* ws,
                         const int* group_off, int groups, hipStream_t st) {
-  if (EPI == EPI_SILU && N % 32) return (int)hipErrorInvalidValue;
+  if (epi_pairs(EPI) && N % 32) return (int)hipErrorInvalidValue;
   const int tiles = ((M + 255) / 256) * ((N + 127) / 128);
   int ksl = K / splits;
   ksl = (ksl / BK) * BK;
@@ -897,7 +900,7 @@ static int launch_8p128(const void* A, int lda, const void* W, int ldw, void* C,
                                                 M, N, K, ksl, (const u16*)bias, (float*)ws,
                                                 group_off);
   if (splits > 1 && C != nullptr) {
-    const int outN = (EPI == EPI_SILU) ? N / 2 : N;
+    const int outN = epi_pairs(EPI) ? N / 2 : N;
     const long total = (long)M * outN;
     splitk_reduce_kernel<EPI><<<(int)((total + 255) / 256), 256, 0, st>>>(
         C, ldc, (const float*)ws, M, N, splits, (const u16*)bias);

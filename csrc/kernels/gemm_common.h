@@ -17,7 +17,12 @@ enum { EPI_BF16 = 0, EPI_F32 = 1, EPI_SILU = 2, EPI_BIAS_GELU = 3, EPI_BIAS = 4,
        // reads; the scale keeps |partial| up to ~1e6 in range). Tiles and 8-phase families.
        EPI_SLAB16 = 5,
        // the exact (erf) GELU of the product, no bias (ungated expert feed-forwards)
-       EPI_GELU_ERF = 6 };
+       EPI_GELU_ERF = 6,
+       // g sigmoid(1.702 g) (u + 1) over the interleaved gate/up weight, g = min(gate, L), u =
+       // clamp(up, -L, L); `bias` points to the fp32 constant L on the device
+       EPI_CLAMP = 7 };
+// epilogues that pair a gate block with the up block beside it (output width N / 2)
+constexpr bool epi_pairs(int epi) { return epi == EPI_SILU || epi == EPI_CLAMP; }
 
 typedef __attribute__((address_space(3))) void lds_void;
 typedef const __attribute__((address_space(1))) void gbl_void;
@@ -192,17 +197,31 @@ __device__ __forceinline__ void store_quad(void* C, int ldc, int row, int col, i
 // of 4, C (and the bias) 16-B (fp32) / 8-B (bf16) aligned (C may be a column view)
 template <int EPI>
 __device__ __forceinline__ bool out_vec(const void* C, int ldc, int N, const u16* bias) {
-  const uintptr_t mis = ((uintptr_t)C | (uintptr_t)bias) & (EPI == EPI_F32 ? 15 : 7);
+  const uintptr_t mis = ((uintptr_t)C | (EPI == EPI_CLAMP ? 0 : (uintptr_t)bias)) & (EPI == EPI_F32 ? 15 : 7);
   return ((N | ldc) & 3) == 0 && mis == 0;
 }
 
-// SiLU(gate) * up of one gate block g and its up block u (same lane, same row): the four
-// features [f, f + 4) of the 16-row-interleaved gate/up layout
-__device__ __forceinline__ void store_silu_quad(void* C, int ldc, int row, int f, f32x4 g,
-                                                f32x4 u, bool vec) {
+__device__ __forceinline__ float clamp_swish_f(float g, float u, float lim) {
+  g = fminf(g, lim);
+  u = fminf(fmaxf(u, -lim), lim);
+  return g / (1.f + __expf(-1.702f * g)) * (u + 1.f);
+}
+template <int EPI> __device__ __forceinline__ float pair_f(float g, float u, float lim) {
+  return EPI == EPI_CLAMP ? clamp_swish_f(g, u, lim) : silu_f(g) * u;
+}
+// the constant of a pairing epilogue
+template <int EPI> __device__ __forceinline__ float pair_const(const u16* bias) {
+  return EPI == EPI_CLAMP ? *reinterpret_cast<const float*>(bias) : 0.f;
+}
+
+// SiLU(gate) * up (or the clamped swish) of one gate block g and its up block u (same lane,
+// same row): the four features [f, f + 4) of the 16-row-interleaved gate/up layout
+template <int EPI = EPI_SILU>
+__device__ __forceinline__ void store_pair_quad(void* C, int ldc, int row, int f, f32x4 g,
+                                                f32x4 u, bool vec, float lim = 0.f) {
   float o[4];
 #pragma unroll
-  for (int r = 0; r < 4; ++r) o[r] = silu_f(g[r]) * u[r];
+  for (int r = 0; r < 4; ++r) o[r] = pair_f<EPI>(g[r], u[r], lim);
   u16* p = (u16*)C + (long)row * ldc + f;
   if (vec) {
     uint2 pk;
@@ -258,16 +277,16 @@ static __global__ void __launch_bounds__(256) splitk_reduce_kernel(void* __restr
                                                             const float* __restrict__ ws, int M,
                                                             int N, int splits,
                                                             const u16* __restrict__ bias) {
-  const int outN = (EPI == EPI_SILU) ? N / 2 : N;
+  const int outN = epi_pairs(EPI) ? N / 2 : N;
   const long gid = (long)blockIdx.x * blockDim.x + threadIdx.x;
   if (gid >= (long)M * outN) return;
   const int row = (int)(gid / outN), col = (int)(gid % outN);
-  if (EPI == EPI_SILU) {
+  if (epi_pairs(EPI)) {
     const int grp = col >> 4, in = col & 15;
     const long gi = (long)row * N + grp * 32 + in, ui = gi + 16;
     float g = 0.f, u = 0.f;
     for (int s = 0; s < splits; ++s) { g += ws[(long)s * M * N + gi]; u += ws[(long)s * M * N + ui]; }
-    ((u16*)C)[(long)row * ldc + col] = f2bf(silu_f(g) * u);
+    ((u16*)C)[(long)row * ldc + col] = f2bf(pair_f<EPI>(g, u, pair_const<EPI>(bias)));
   } else {
     float v = 0.f;
     for (int s = 0; s < splits; ++s) v += ws[(long)s * M * N + (long)row * N + col];
@@ -296,6 +315,7 @@ int gemm_4w_set_slab_store(int mode);
 // EPI -> template argument, for a family's dispatch<EPI>(tile_cfg, ...); the families with
 // an fp16 slab store (tiles, 8-phase) take DLI_EPI_SWITCH_S16
 #define DLI_EPI_SWITCH_S16(FN)                                                     \
+  if (epi == EPI_CLAMP) return FN<EPI_CLAMP>(tile_cfg, DLI_GEMM_PASS);             \
   if (epi == EPI_SLAB16) {                                                         \
     if (C != nullptr || splits < 2) return (int)hipErrorInvalidValue;              \
     return FN<EPI_SLAB16>(tile_cfg, DLI_GEMM_PASS);                                \

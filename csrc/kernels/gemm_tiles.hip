@@ -180,7 +180,8 @@ __global__ void __launch_bounds__(64 * WM * WN) gemm_bf16_kernel(
     return;
   }
   const bool vec = out_vec<EPI>(C, ldc, N, bias);
-  if (EPI == EPI_SILU) {
+  if (epi_pairs(EPI)) {
+    const float lim = pair_const<EPI>(bias);
     // column blocks j (even) = gate, j+1 = up of the same 16 features
 #pragma unroll
     for (int i = 0; i < MI; ++i) {
@@ -190,8 +191,8 @@ __global__ void __launch_bounds__(64 * WM * WN) gemm_bf16_kernel(
       for (int j = 0; j < NI; j += 2) {
         const int gcol = n0 + wn * TN + 16 * j;         // first gate row of the pair
         if (gcol < N)
-          store_silu_quad(C, ldc, row0 + row, (gcol >> 5) * 16 + 4 * fq, acc[i][j],
-                          acc[i][j + 1], vec);
+          store_pair_quad<EPI>(C, ldc, row0 + row, (gcol >> 5) * 16 + 4 * fq, acc[i][j],
+                          acc[i][j + 1], vec, lim);
       }
     }
     return;
@@ -212,7 +213,7 @@ template <int BM, int BN, int EPI, int NS, int WM = 2, int WN = 2>
 static int launch_cfg(const void* A, int lda, const void* W, int ldw, void* C, int ldc, int M,
                       int N, int K, int splits, const void* bias, void* ws,
                       const int* group_off, int groups, hipStream_t st) {
-  if (EPI == EPI_SILU && (BN / WN) % 32) return (int)hipErrorInvalidValue;  // gate/up pairs
+  if (epi_pairs(EPI) && (BN / WN) % 32) return (int)hipErrorInvalidValue;  // gate/up pairs
   const int tiles = ((M + BM - 1) / BM) * ((N + BN - 1) / BN);
   int ksl = K / splits;
   ksl = (ksl / BK) * BK;
@@ -229,7 +230,7 @@ static int launch_cfg(const void* A, int lda, const void* W, int ldw, void* C, i
       (const u16*)A, lda, (const u16*)W, ldw, C, ldc, M, N, K, ksl, (const u16*)bias,
       (float*)ws, group_off);
   if (splits > 1 && C != nullptr) {       // C == nullptr: leave the fp32 partial slabs for a
-    const int outN = (EPI == EPI_SILU) ? N / 2 : N;   // fused consumer (fused_reduce.hip)
+    const int outN = epi_pairs(EPI) ? N / 2 : N;   // fused consumer (fused_reduce.hip)
     const long total = (long)M * outN;
     splitk_reduce_kernel<EPI><<<(int)((total + 255) / 256), 256, 0, st>>>(
         C, ldc, (const float*)ws, M, N, splits, (const u16*)bias);

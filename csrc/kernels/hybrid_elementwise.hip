@@ -53,30 +53,41 @@ __global__ void __launch_bounds__(256) embedding_f32_kernel(
   if (x0 != nullptr) x0[gid] = v;
 }
 
-// One workgroup per row. x (fp32, in place): x = keep * x + mult * y + bias + add, y, bias and
-// the rows `add` (fp32, x's layout) may be null. The row is cut into `groups` equal parts, each scaled by its own rsqrt(mean(sq) + eps);
-// h = that * w. h may be null (the last layer's add). rows_idx (nullable) selects source rows
-// (the final norm of the rows whose logits are wanted); it excludes y / bias / the write-back.
+// One workgroup per row (256 threads; 1024 for the few wide rows of a decode step, which are
+// bound by latency). x (fp32, in place): x = keep * x + mult * y + bias + add, y, bias and the
+// rows `add` (fp32, x's layout) may be null. y may be nsplit slabs, ysplit elements apart, of a
+// split-K GEMM: they are summed here, in order. The row is cut into `groups` equal parts, each
+// scaled by its own rsqrt(mean(sq) + eps); h = that * w. h may be null (the last layer's add).
+// rows_idx (nullable) selects source rows (the final norm of the rows whose logits are
+// wanted); it excludes y / bias / add / the write-back.
 template <typename S>
-__global__ void __launch_bounds__(256) resadd_groupnorm_kernel(
-    float* __restrict__ x, const float* __restrict__ y, int ldy, const S* __restrict__ bias,
-    const float* __restrict__ add, float keep, float mult, const S* __restrict__ w,
-    void* __restrict__ h, int ldh, int dim, int groups, float eps, const long* __restrict__ rows_idx, bool vec4, float gain,
-    bool h_f32, float w_offset) {
+__global__ void __launch_bounds__(1024) resadd_groupnorm_kernel(
+    float* __restrict__ x, const float* __restrict__ y, int ldy, int nsplit, long ysplit,
+    const S* __restrict__ bias, const float* __restrict__ add, float keep, float mult,
+    const S* __restrict__ w, void* __restrict__ h, int ldh, int dim, int groups, float eps,
+    const long* __restrict__ rows_idx, bool vec4, float gain, bool h_f32, float w_offset) {
   extern __shared__ __attribute__((aligned(16))) float row[];   // dim floats + group scales
+  __shared__ float red[16];
   float* gsum = row + dim;
   const int r = blockIdx.x;
   const long src = rows_idx ? rows_idx[r] : r;
   float* xr = x + src * dim;
-  for (int g = threadIdx.x; g < groups; g += blockDim.x) gsum[g] = 0.f;
-  const bool update = rows_idx == nullptr && (y != nullptr || bias != nullptr || add != nullptr || keep != 1.f);
+  const bool update = rows_idx == nullptr &&
+                      (y != nullptr || bias != nullptr || add != nullptr || keep != 1.f);
+  float ss = 0.f;                           // of this thread's columns
   if (vec4) {                               // 16-byte loads and stores of the fp32 rows
     for (int c = threadIdx.x * 4; c < dim; c += blockDim.x * 4) {
       f32x4 v = *reinterpret_cast<const f32x4*>(xr + c);
       if (rows_idx == nullptr) {
         if (keep == 0.f) v = f32x4{0.f, 0.f, 0.f, 0.f};
         else if (keep != 1.f) v *= keep;
-        if (y != nullptr) v += mult * *reinterpret_cast<const f32x4*>(y + (long)r * ldy + c);
+        if (y != nullptr) {
+          const float* yp = y + (long)r * ldy + c;
+          f32x4 t = *reinterpret_cast<const f32x4*>(yp);
+#pragma unroll 4
+          for (int k = 1; k < nsplit; ++k) t += *reinterpret_cast<const f32x4*>(yp + k * ysplit);
+          v += mult * t;
+        }
         if (bias != nullptr) {
 #pragma unroll
           for (int u = 0; u < 4; ++u) v[u] += ldf(bias + c + u);
@@ -85,32 +96,62 @@ __global__ void __launch_bounds__(256) resadd_groupnorm_kernel(
         if (update) *reinterpret_cast<f32x4*>(xr + c) = v;
       }
       *reinterpret_cast<f32x4*>(row + c) = v;
+      ss += (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]);
     }
   } else {
     for (int c = threadIdx.x; c < dim; c += blockDim.x) {
       float v = xr[c];
       if (rows_idx == nullptr) {
         v = keep != 0.f ? v * keep : 0.f;
-        if (y != nullptr) v += mult * y[(long)r * ldy + c];
+        if (y != nullptr) {
+          float t = y[(long)r * ldy + c];
+          for (int k = 1; k < nsplit; ++k) t += y[(long)r * ldy + c + k * ysplit];
+          v += mult * t;
+        }
         if (bias != nullptr) v += ldf(bias + c);
         if (add != nullptr) v += add[(long)r * dim + c];
         if (update) xr[c] = v;
       }
       row[c] = v;
+      ss += v * v;
+    }
+  }
+  if (h == nullptr) return;
+  const int gl = dim / groups;
+  if (groups == 1) {
+    const float tot = block_sum(ss, red);
+    if (threadIdx.x == 0) gsum[0] = 1.f / sqrtf(tot / (float)dim + eps);
+  } else {
+    __syncthreads();
+    // one wave per group, in turn: a wave sums its group's squares in a fixed order
+    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, nw = blockDim.x >> 6;
+    for (int g = wid; g < groups; g += nw) {
+      float s = 0.f;
+      for (int c = lane; c < gl; c += 64) { const float v = row[g * gl + c]; s += v * v; }
+      s = wave_sum(s);
+      if (lane == 0) gsum[g] = 1.f / sqrtf(s / (float)gl + eps);
     }
   }
   __syncthreads();
-  if (h == nullptr) return;
-  const int gl = dim / groups;
-  // one wave per group, in turn: a wave sums its group's squares in a fixed order
-  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, nw = blockDim.x >> 6;
-  for (int g = wid; g < groups; g += nw) {
-    float s = 0.f;
-    for (int c = lane; c < gl; c += 64) { const float v = row[g * gl + c]; s += v * v; }
-    s = wave_sum(s);
-    if (lane == 0) gsum[g] = 1.f / sqrtf(s / (float)gl + eps);
+  if (vec4 && !h_f32 && groups == 1 && ldh % 4 == 0) {
+    const float rs = gsum[0] * gain;
+    for (int c = threadIdx.x * 4; c < dim; c += blockDim.x * 4) {
+      const f32x4 v = *reinterpret_cast<const f32x4*>(row + c);
+      float o[4];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) o[u] = v[u] * rs * (ldf(w + c + u) + w_offset);
+      S* hp = (S*)h + (long)r * ldh + c;
+      if constexpr (sizeof(S) == 2) {
+        uint2 pk;
+        pk.x = pack2bf(o[0], o[1]);
+        pk.y = pack2bf(o[2], o[3]);
+        *reinterpret_cast<uint2*>(hp) = pk;
+      } else {
+        *reinterpret_cast<f32x4*>(hp) = f32x4{o[0], o[1], o[2], o[3]};
+      }
+    }
+    return;
   }
-  __syncthreads();
   if (h_f32) {
     for (int c = threadIdx.x; c < dim; c += blockDim.x)
       ((float*)h)[(long)r * ldh + c] = row[c] * gsum[c / gl] * (ldf(w + c) + w_offset) * gain;
@@ -425,25 +466,26 @@ extern "C" int dli_embedding_f32(float* x, float* x0, const int* ids, const void
   DLI_RETURN_LAUNCH();
 }
 
-extern "C" int dli_resadd_groupnorm(float* x, const float* y, int ldy, const void* bias,
-                                    const float* add, float keep, float mult, const void* w,
-                                    void* h, int ldh, int rows, int dim, int groups, float eps,
-                                    const long* rows_idx, float gain, int h_f32, float w_offset,
-                                    int dt, hipStream_t st) {
+extern "C" int dli_resadd_groupnorm(float* x, const float* y, int ldy, int nsplit, long ysplit,
+                                    const void* bias, const float* add, float keep, float mult,
+                                    const void* w, void* h, int ldh, int rows, int dim, int groups,
+                                    float eps, const long* rows_idx, float gain, int h_f32,
+                                    float w_offset, int dt, hipStream_t st) {
   if (rows <= 0) return 0;
-  if (groups < 1 || dim % groups || (size_t)(dim + groups) * 4 > 60000)
+  if (groups < 1 || dim % groups || (size_t)(dim + groups) * 4 > 60000 || nsplit < 1)
     return (int)hipErrorInvalidValue;
   const size_t sh = (size_t)(dim + groups) * 4;
-  const bool vec4 = dim % 4 == 0 && (uintptr_t)x % 16 == 0 &&
-                    (y == nullptr || ((uintptr_t)y % 16 == 0 && ldy % 4 == 0)) &&
+  const bool vec4 = dim % 4 == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)h % 16 == 0 &&
+                    (y == nullptr || ((uintptr_t)y % 16 == 0 && ldy % 4 == 0 && ysplit % 4 == 0)) &&
                     (uintptr_t)add % 16 == 0;
+  const int nt = (rows <= 1024 && dim >= 2048) ? 1024 : 256;
   DT_SWITCH(dt,
-            (resadd_groupnorm_kernel<u16><<<rows, 256, sh, st>>>(
-                x, y, ldy, (const u16*)bias, add, keep, mult, (const u16*)w, h, ldh, dim, groups,
-                eps, rows_idx, vec4, gain, h_f32 != 0, w_offset)),
-            (resadd_groupnorm_kernel<float><<<rows, 256, sh, st>>>(
-                x, y, ldy, (const float*)bias, add, keep, mult, (const float*)w, h, ldh, dim,
-                groups, eps, rows_idx, vec4, gain, h_f32 != 0, w_offset)));
+            (resadd_groupnorm_kernel<u16><<<rows, nt, sh, st>>>(
+                x, y, ldy, nsplit, ysplit, (const u16*)bias, add, keep, mult, (const u16*)w, h,
+                ldh, dim, groups, eps, rows_idx, vec4, gain, h_f32 != 0, w_offset)),
+            (resadd_groupnorm_kernel<float><<<rows, nt, sh, st>>>(
+                x, y, ldy, nsplit, ysplit, (const float*)bias, add, keep, mult, (const float*)w,
+                h, ldh, dim, groups, eps, rows_idx, vec4, gain, h_f32 != 0, w_offset)));
   DLI_RETURN_LAUNCH();
 }
 

@@ -267,6 +267,8 @@ class HybridLM(TransformerLM):
             if "ff_tuned" in lp:
                 if spec.ff_kind == "gelu":
                     fused[id(lp["w_up"])] = "bias_gelu"
+                elif spec.ff_kind == "clamp_swish":
+                    fused[id(lp["w_gu"])] = "clamp_mul"
                 elif spec.ff_kind == "gated_silu":
                     fused[id(lp["w_gu"])] = "silu_mul"
                 elif spec.shared_ff and spec.expert_act == "gelu_erf":

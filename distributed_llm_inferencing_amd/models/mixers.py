@@ -254,7 +254,7 @@ def retention_mixer(spec: LayerSpec, lp: dict, h, step: StepView, cache, eps: fl
     o = H.retention(proj, step.rotation(spec, lp), spec.rot_dims, lp["decay_pow"], eps, state,
                     step.state_slots, step.cu_seqlens, step.max_seqlen, step.positions,
                     spec.heads, spec.dim, spec.vdim, h.dtype)
-    return H.linear_any(o, lp["wo"])
+    return H.linear_out(o, lp["wo"])
 
 
 def rope_attention_mixer(spec: LayerSpec, lp: dict, h, step: StepView, cache, eps: float):
@@ -273,7 +273,7 @@ def rope_attention_mixer(spec: LayerSpec, lp: dict, h, step: StepView, cache, ep
                            step.cu_seqlens, step.max_seqlen, step.positions, step.block_tables,
                            step.block_size, win, spec.scale,
                            keep_first=min(spec.keep_first, ctx) if win < ctx else 0)
-    return H.linear_any(o, lp["wo"])
+    return H.linear_out(o, lp["wo"])
 
 
 MIXERS = {"attention": attention_mixer, "hgrn2": hgrn2_mixer,
@@ -286,7 +286,7 @@ MIXERS = {"attention": attention_mixer, "hgrn2": hgrn2_mixer,
 # Two layouts of a feed-forward's weights. The plain one ([gate | up] stacked) runs the
 # shape-agnostic GEMM with fp32 outputs and separate activation kernels: any sizes, bf16 or
 # fp32. The tuned one (``prepare_feed_forward``: bf16, sizes the tile family takes) fuses the
-# activation into the first GEMM's epilogue — SiLU * up over the 16-row interleaved gate/up
+# activation into the first GEMM's epilogue — SiLU * up or the clamped swish over the 16-row interleaved gate/up
 # weight, bias + GELU for the ungated form — and runs the experts as the grouped GEMMs of the
 # framework's other mixture model.
 def prepare_feed_forward(spec: LayerSpec, params: dict, pre: str) -> None:
@@ -297,12 +297,15 @@ def prepare_feed_forward(spec: LayerSpec, params: dict, pre: str) -> None:
     from ..ops.reference import interleave_gate_up
     w = params.get(pre + "w_down")
     if (not spec.ff or w is None or pre + "ff_tuned" in params or w.dtype != torch.bfloat16
-            or not w.is_cuda or spec.ff_kind not in ("gelu", "moe", "gated_silu")
+            or not w.is_cuda or spec.ff_kind not in ("gelu", "moe", "gated_silu", "clamp_swish")
             or w.shape[-2] % 64 or spec.ff % 64 or spec.shared_ff % 64):
         return
     if spec.ff_kind == "gelu":
         params[pre + "b_up"] = torch.zeros(spec.ff, dtype=w.dtype, device=w.device)
-    elif spec.ff_kind == "gated_silu":
+    elif spec.ff_kind in ("gated_silu", "clamp_swish"):
+        if spec.ff_kind == "clamp_swish":            # read by the GEMM's epilogue
+            params[pre + "act_limit"] = torch.full((1,), spec.act_limit, dtype=torch.float32,
+                                                   device=w.device)
         gu = params[pre + "w_gu"]
         params[pre + "w_gu"] = interleave_gate_up(gu[:spec.ff], gu[spec.ff:]).contiguous()
     elif spec.ff_kind == "moe" and spec.expert_act == "clamp_swish":
@@ -342,9 +345,13 @@ def gated_silu_ff(spec: LayerSpec, lp: dict, h):
 
 def clamp_swish_ff(spec: LayerSpec, lp: dict, h):
     """down(g sigmoid(1.702 g) (u + 1)), g = min(gate, limit), u = clamp(up, -limit, limit)."""
-    act = H.act_mul(H.linear_any(h, lp["w_gu"]), spec.ff, h.dtype, "clamp_swish",
-                    limit=spec.act_limit)
-    return H.linear_any(act, lp["w_down"])
+    if "ff_tuned" in lp:
+        from .. import ops
+        act = ops.linear(h, lp["w_gu"], lp["act_limit"], epi="clamp_mul")
+    else:
+        act = H.act_mul(H.linear_any(h, lp["w_gu"]), spec.ff, h.dtype, "clamp_swish",
+                        limit=spec.act_limit)
+    return H.linear_out(act, lp["w_down"])
 
 
 def moe_ff(spec: LayerSpec, lp: dict, h):

@@ -221,7 +221,7 @@ def _gemm_native(x, w, epi: str, bias=None, out=None, plan: Optional[G.GemmPlan]
             plan = G.plan(M, Nn, K, epi)
         else:
             plan = G.grouped_plan(M, Nn, K, epi, groups)
-    out_n = Nn // 2 if epi == "silu_mul" else Nn
+    out_n = Nn // 2 if epi in G.PAIR_EPIS else Nn
     if out is None:
         dt = torch.float32 if epi == "f32" else x.dtype
         out = torch.empty(M, out_n, dtype=dt, device=x.device)
@@ -237,8 +237,9 @@ def _gemm_native(x, w, epi: str, bias=None, out=None, plan: Optional[G.GemmPlan]
 
 
 def linear(x, w, bias=None, epi: str = "none", out=None):
-    """y = epi(x @ w.T (+bias)). epi in {none, f32, silu_mul, bias_gelu, bias, gelu_erf}.
-    silu_mul expects the 16-row interleaved gate/up weight and returns width N/2."""
+    """y = epi(x @ w.T (+bias)). epi in {none, f32, silu_mul, bias_gelu, bias, gelu_erf,
+    clamp_mul}. silu_mul and clamp_mul expect the 16-row interleaved gate/up weight and return
+    width N/2; clamp_mul takes its limit as ``bias``, one fp32 number on the device."""
     if bias is not None and epi == "none":
         epi = "bias"
     if isinstance(x, NormedRows):
@@ -257,6 +258,9 @@ def linear(x, w, bias=None, epi: str = "none", out=None):
             y = R.linear(x, w, out_dtype=torch.float32)
         elif epi == "bias_gelu":
             y = R.gelu_tanh(R.linear(x, w, bias))
+        elif epi == "clamp_mul":
+            gu = torch.cat(R.split_gate_up(R.linear(x, w, out_dtype=torch.float32)), -1)
+            y = R.clamp_swish_mul(gu, w.shape[-2] // 2, float(bias), x.dtype)
         elif epi == "gelu_erf":
             y = torch.nn.functional.gelu(R.linear(x, w, out_dtype=torch.float32)).to(x.dtype)
         else:

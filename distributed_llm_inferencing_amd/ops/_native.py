@@ -74,7 +74,7 @@ _SIGS = {
     # hybrid family (ops/hybrid.py)
     "dli_gemm_any": [P, L, P, L, P, L, I, I, I, I, I, I, L, L, L, P],
     "dli_embedding_f32": [P, P, P, P, I, I, I, F, P, P, I, I, P],
-    "dli_resadd_groupnorm": [P, P, I, P, P, F, F, P, P, I, I, I, I, F, P, F, I, F, I, P],
+    "dli_resadd_groupnorm": [P, P, I, I, L, P, P, F, F, P, P, I, I, I, I, F, P, F, I, F, I, P],
     "dli_token_shift": [P, P, P, P, P, P, P, I, I, I, I, P],
     "dli_act_mul": [P, I, P, I, I, I, I, P, F, I, I, P],
     "dli_talk_prepare": [P, I, P, P, F, I, I, I, I, I, P, P, P, P, I, P],

@@ -88,13 +88,13 @@ def tile_ok(tile: int, epi: str) -> bool:
     which must therefore be a multiple of 32."""
     if epi == "res":
         return tile in GEMV_RES_TILES
-    if epi == "gelu_erf" and tile in (34, 41, 45, 55):
-        return False            # the 4-wave families are built without the exact-GELU epilogue
+    if epi in ("gelu_erf", "clamp_mul") and tile in (34, 41, 45, 55):
+        return False            # the 4-wave families are built without these epilogues
     if tile in (29, 58, 59):
         return epi == "silu_mul"
     if tile in GEMV_TILES:
-        return epi != "silu_mul" or tile in (31, 33)
-    if epi != "silu_mul":
+        return epi != "clamp_mul" and (epi != "silu_mul" or tile in (31, 33))
+    if epi not in PAIR_EPIS:
         return True
     if tile == 26:              # the straddling gate/up pair meets through LDS
         return True
@@ -105,7 +105,9 @@ def tile_ok(tile: int, epi: str) -> bool:
 # "splitk": a plain GEMM whose fp32 partial slabs feed a fused reduce (ops.linear_add_rmsnorm,
 # ops.linear_rope_cache); planned/tuned separately (a non-split winner runs unfused).
 EPI = {"none": 0, "f32": 1, "silu_mul": 2, "bias_gelu": 3, "bias": 4, "splitk": 0,
-       "slab16": 5, "gelu_erf": 6}
+       "slab16": 5, "gelu_erf": 6, "clamp_mul": 7}
+# epilogues over the interleaved gate/up weight: the output is half as wide
+PAIR_EPIS = ("silu_mul", "clamp_mul")
 # tiles whose slab-only split-K call can store fp16 partials (EPI "slab16": the generic tile
 # family and the 8-phase kernels); the fused consumers then read half the bytes. The
 # weight-streaming GEMVs and the 4-wave family keep fp32 slabs.
@@ -174,7 +176,7 @@ def _heuristic(M: int, N: int, K: int, epi: str) -> GemmPlan:
         # residual-adding GEMV (full K): 4 rows a workgroup, 8 K-steps in flight per lane
         # (1024 workgroups on a 4096-wide projection)
         return GemmPlan("dli", 56, 1)
-    if M <= GEMV_MAX_M:
+    if M <= GEMV_MAX_M and epi != "clamp_mul":      # (the GEMVs are built without it)
         # batch-1 / tiny batches: stream the weights (gemv_kernel) with enough workgroups
         # (>= 512, two per CU) to keep ~64 KB of loads in flight per CU
         # gate/up at M <= 2: the 16-row SiLU grid (tile 29) 39.5 / 43.3 vs 49.0 / 51.0 us for
@@ -380,6 +382,7 @@ def autotune(shapes, weights: dict, device, iters: int = 6, log=None,
                 bt = (slots // 16).to(torch.int32).unsqueeze(1).contiguous()
                 ctx = torch.ones(M, dtype=torch.int32, device=device)
                 sc = 1.0 / math.sqrt(hd)
+        bias = (torch.ones(1, dtype=torch.float32, device=device) if epi == "clamp_mul" else None)
         best = None
         timed = []                                  # (ms, plan, run) of every valid candidate
         t_shape = time.perf_counter()
@@ -399,7 +402,7 @@ def autotune(shapes, weights: dict, device, iters: int = 6, log=None,
                     elif epi == "res":
                         ops.linear_residual(x, w, res_r, plan=p)
                     else:
-                        ops._gemm_native(x, w, epi, plan=p)
+                        ops._gemm_native(x, w, epi, bias=bias, plan=p)
             try:
                 ms = ops.benchmark(run, iters=iters, warmup=1, graph=_GRAPH_TUNE) / len(ws_)
             except Exception:  # noqa: BLE001 — an invalid candidate is skipped

@@ -69,6 +69,33 @@ def linear_any(x: torch.Tensor, w: torch.Tensor, out_f32: bool = True,
     return out
 
 
+def linear_out(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """x @ w^T in fp32 for a consumer that adds it to the residual (``resadd_groupnorm``, or any
+    through ``rows_of``): [M, N], or, where the planned GEMM splits K, its partial sums
+    [splits, M, N] in the shared workspace, which the add sums itself (one launch and one pass
+    less). They must be consumed before the next GEMM."""
+    if (x.is_cuda and x.dtype == torch.bfloat16 and x.shape[1] % 64 == 0 and w.shape[0] % 4 == 0
+            and x.stride(0) % 8 == 0 and w.stride(0) % 8 == 0 and x.stride(1) == 1
+            and w.stride(1) == 1 and x.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0):
+        (M, K), Nn = x.shape, w.shape[0]
+        p = _gemm.plan(M, Nn, K, "f32")
+        if p.splits > 1:
+            ws = _gemm.workspace(x.device, p.splits * M * Nn * 4)
+            _call("dli_gemm", _p(x), x.stride(0), _p(w), w.stride(0), None, Nn, M, Nn, K,
+                  _gemm.EPI["f32"], p.tile, p.splits, None, _p(ws), None, 1, _st())
+            return ws[:p.splits * M * Nn * 4].view(torch.float32).view(p.splits, M, Nn)
+    return linear_any(x, w)
+
+
+def rows_of(y: Optional[torch.Tensor]) -> Optional[torch.Tensor]:
+    """[M, N] from what ``linear_out`` returned."""
+    if y is None or y.dim() == 2:
+        return y
+    x = torch.empty(y.shape[1:], dtype=torch.float32, device=y.device)
+    resadd_groupnorm(x, y, None, 1, 0.0, keep=0.0)
+    return x
+
+
 def head_linear(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
     """Per-head projection: out[:, h, :n] = x[:, h, :] @ w[h]^T for x [T, H, k], w [H, n, k],
     out [T, H, >= n] (the result lands in the first n columns of each head's row; x and out may
@@ -113,7 +140,7 @@ def resadd_groupnorm(x: torch.Tensor, y: Optional[torch.Tensor], w: Optional[tor
                      out_f32: bool = False, w_offset: float = 0.0,
                      add: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
     """In place on the fp32 stream: x = keep * x + mult * y + bias + add (y, bias and the fp32
-    rows ``add`` optional); returns
+    rows ``add`` optional; y may be a GEMM's partial sums, see ``linear_out``); returns
     the grouped RMS norm of the new x times ``w`` times ``gain`` in the storage dtype (None when
     w is None), or unrounded in fp32 with ``out_f32`` (what a token shift reads). ``w_offset``
     is added to the weight in fp32 (weights stored as offsets from one)."""
@@ -139,8 +166,9 @@ def resadd_groupnorm(x: torch.Tensor, y: Optional[torch.Tensor], w: Optional[tor
          if w is not None else None)
     if add is not None and (add.shape != x.shape or not add.is_contiguous()):
         raise ValueError("resadd_groupnorm: add must have the stream's shape")
-    _call("dli_resadd_groupnorm", _p(x), _p(y), y.stride(0) if y is not None else 0, _p(bias),
-          _p(add), float(keep), float(mult), _p(w), _p(h), dim, rows, dim, groups, float(eps), None,
+    slabs = y is not None and y.dim() == 3
+    _call("dli_resadd_groupnorm", _p(x), _p(y), y.stride(-2) if y is not None else 0,
+          y.shape[0] if slabs else 1, y.stride(0) if slabs else 0, _p(bias), _p(add), float(keep), float(mult), _p(w), _p(h), dim, rows, dim, groups, float(eps), None,
           float(gain), int(out_f32), float(w_offset), _dt(dtype), _st())
     return h
 
@@ -153,7 +181,7 @@ def groupnorm_rows(x: torch.Tensor, rows_idx: torch.Tensor, w: torch.Tensor, gro
         return (h * gain if gain != 1.0 else h).to(w.dtype)
     n, dim = rows_idx.shape[0], x.shape[1]
     h = torch.empty(n, dim, dtype=w.dtype, device=x.device)
-    _call("dli_resadd_groupnorm", _p(x), None, 0, None, None, 1.0, 1.0, _p(w), _p(h), dim, n, dim,
+    _call("dli_resadd_groupnorm", _p(x), None, 0, 1, 0, None, None, 1.0, 1.0, _p(w), _p(h), dim, n, dim,
           groups, float(eps), _p(rows_idx), float(gain), 0, float(w_offset), _dt(w.dtype), _st())
     return h
 
@@ -470,6 +498,7 @@ def postnorm(x, y, w, b, eps: float, keep: float = 1.0,
     """x = LayerNorm(keep * x + y) * w + b on the fp32 stream, in place (y optional, fp32);
     returns the new rows in the storage dtype (w's). With ``rows_idx`` (int64) only those rows
     are normed and returned and x is left alone."""
+    y = rows_of(y)
     if not x.is_cuda:
         return R.postnorm(x, y, w, b, eps, keep, w.dtype, rows_idx)
     dim = x.shape[1]
@@ -636,6 +665,7 @@ def hyper_mix(xs, y, prev, read, w, eps: float = 0.0, w_offset: float = 0.0, dty
     fp32 vector read | write | mix) the streams are mixed and receive y; with ``read`` (the next
     sublayer's vector, or ones for the plain sum) the weighted sum of the new streams is
     returned — RMS-normed times (w + w_offset) in the storage dtype when w is given, else fp32."""
+    y = rows_of(y)
     if not xs.is_cuda:
         return R.hyper_mix(xs, y, prev, read, w, eps, w_offset, dtype or (w.dtype if w is not None else None))
     T, S, D = xs.shape

@@ -335,6 +335,51 @@ def test_clamped_feed_forward(device, dtype, ff, limit):
         assert (g > limit).any() and (u > limit).any() and (u < -limit).any()
 
 
+@pytest.mark.gpu
+@pytest.mark.parametrize("M,splits", [(3, 2), (40, 4), (130, 2)])
+def test_residual_add_sums_the_partial_sums_of_a_split_gemm(M, splits):
+    from distributed_llm_inferencing_amd.ops import gemm as G
+    N, K, eps = 192, 512, 1e-5
+    x, w = hidden(M, K, 1), O.bf16_exact(hidden(N, K, 2) / 20)
+    base, b, nw = hidden(M, N, 3), hidden(1, N, 4)[0], hidden(1, N, 5)[0]
+    key = (G._bucket(M), N, K, "f32")
+    old = G._plan_cache.get(key)
+    G.set_plan(M, N, K, "f32", G.GemmPlan("dli", 0, splits))
+    try:
+        bf = torch.bfloat16
+        xt, wt = dev_t(x, "cuda", bf), dev_t(w, "cuda", bf)
+        y = H.linear_out(xt, wt)
+        assert y.shape == (splits, M, N)
+        st = dev_t(base, "cuda")
+        h = H.resadd_groupnorm(st, y, dev_t(nw, "cuda", bf), 1, eps, bias=dev_t(b, "cuda", bf))
+        want = base + x @ w.T + b
+        np.testing.assert_allclose(st.cpu().numpy(), want, atol=2e-4, rtol=2e-4)
+        np.testing.assert_allclose(h.float().cpu().numpy(), O.norm(want, nw, eps), atol=3e-2, rtol=3e-2)
+        np.testing.assert_allclose(H.rows_of(H.linear_out(xt, wt)).cpu().numpy(), x @ w.T,
+                                   atol=2e-4, rtol=2e-4)
+    finally:
+        G._plan_cache.pop(key, None) if old is None else G.set_plan(M, N, K, "f32", old)
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("tile,splits", [(0, 1), (0, 2), (1, 4), (2, 1), (13, 1), (22, 1), (22, 2),
+                                         (26, 1), (28, 2)])
+@pytest.mark.parametrize("M", [5, 70, 300])
+def test_clamped_swish_in_the_gemm_epilogue(tile, splits, M):
+    from distributed_llm_inferencing_amd import ops
+    from distributed_llm_inferencing_amd.ops import gemm as G
+    from distributed_llm_inferencing_amd.ops.reference import interleave_gate_up
+    F, K, lim = 448, 256, 0.8
+    x, g, u = hidden(M, K, 1), O.bf16_exact(hidden(F, K, 2) / 12), O.bf16_exact(hidden(F, K, 3) / 12)
+    bf = torch.bfloat16
+    gu = interleave_gate_up(dev_t(g, "cuda", bf), dev_t(u, "cuda", bf)).contiguous()
+    got = ops._gemm_native(dev_t(x, "cuda", bf), gu, "clamp_mul",
+                           bias=torch.full((1,), lim, device="cuda"), plan=G.GemmPlan("dli", tile, splits))
+    w = {"gate": g, "up": u, "down": np.eye(F)}
+    want = O.dense_ff(x, w, "", lim)
+    np.testing.assert_allclose(got.float().cpu().numpy(), want, atol=2e-2, rtol=2e-2)
+
+
 # ------------------------------------------------------------------ whole models
 @pytest.mark.parametrize("device,dtype", CASES)
 @pytest.mark.parametrize("lay", [retention(), retention(mlp=dense()), attention(),
