@@ -33,24 +33,36 @@ template <typename S> __device__ __forceinline__ void stf(S* p, float v);
 template <> __device__ __forceinline__ void stf<u16>(u16* p, float v) { *p = f2bf(v); }
 template <> __device__ __forceinline__ void stf<float>(float* p, float v) { *p = v; }
 
-template <typename S>
+// VEC = 4: rows of a multiple of 4 columns, 16-byte stores
+template <typename S, int VEC>
 __global__ void __launch_bounds__(256) embedding_f32_kernel(
     float* __restrict__ x, float* __restrict__ x0, const int* __restrict__ ids,
     const S* __restrict__ table, int T, int dim, int vocab, float scale,
     const S* __restrict__ pos_table, const int* __restrict__ positions, int max_pos) {
   const long gid = (long)blockIdx.x * blockDim.x + threadIdx.x;
-  if (gid >= (long)T * dim) return;
-  const int t = (int)(gid / dim), c = (int)(gid % dim);
+  const int w = dim / VEC;
+  if (gid >= (long)T * w) return;
+  const int t = (int)(gid / w), c = (int)(gid - (long)t * w) * VEC;
   int id = ids[t];
   id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
-  float v = ldf(table + (long)id * dim + c) * scale;
+  float v[VEC];
+#pragma unroll
+  for (int u = 0; u < VEC; ++u) v[u] = ldf(table + (long)id * dim + c + u) * scale;
   if (pos_table != nullptr) {
     int p = positions[t];
     p = p < 0 ? 0 : (p >= max_pos ? max_pos - 1 : p);
-    v += ldf(pos_table + (long)p * dim + c);
+#pragma unroll
+    for (int u = 0; u < VEC; ++u) v[u] += ldf(pos_table + (long)p * dim + c + u);
   }
-  x[gid] = v;
-  if (x0 != nullptr) x0[gid] = v;
+  const long o = (long)t * dim + c;
+  if constexpr (VEC == 4) {
+    const f32x4 q = {v[0], v[1], v[2], v[3]};
+    *reinterpret_cast<f32x4*>(x + o) = q;
+    if (x0 != nullptr) *reinterpret_cast<f32x4*>(x0 + o) = q;
+  } else {
+    x[o] = v[0];
+    if (x0 != nullptr) x0[o] = v[0];
+  }
 }
 
 // One workgroup per row (256 threads; 1024 for the few wide rows of a decode step, which are
@@ -454,15 +466,14 @@ extern "C" int dli_embedding_f32(float* x, float* x0, const int* ids, const void
   if (T <= 0) return 0;
   if (pos_table != nullptr && (positions == nullptr || max_pos < 1))
     return (int)hipErrorInvalidValue;
-  const int nb = (int)(((long)T * dim + 255) / 256);
-  DT_SWITCH(dt,
-            (embedding_f32_kernel<u16><<<nb, 256, 0, st>>>(x, x0, ids, (const u16*)table, T, dim,
-                                                          vocab, scale, (const u16*)pos_table,
-                                                          positions, max_pos)),
-            (embedding_f32_kernel<float><<<nb, 256, 0, st>>>(x, x0, ids, (const float*)table, T,
-                                                            dim, vocab, scale,
-                                                            (const float*)pos_table, positions,
-                                                            max_pos)));
+  const bool v4 = dim % 4 == 0 && (((uintptr_t)x | (uintptr_t)x0) & 15) == 0;
+  const int nb = (int)(((long)T * (v4 ? dim / 4 : dim) + 255) / 256);
+#define EMB_LAUNCH(S, V)                                                                        \
+  embedding_f32_kernel<S, V><<<nb, 256, 0, st>>>(x, x0, ids, (const S*)table, T, dim, vocab,    \
+                                                 scale, (const S*)pos_table, positions, max_pos)
+  if (v4) DT_SWITCH(dt, EMB_LAUNCH(u16, 4), EMB_LAUNCH(float, 4));
+  else DT_SWITCH(dt, EMB_LAUNCH(u16, 1), EMB_LAUNCH(float, 1));
+#undef EMB_LAUNCH
   DLI_RETURN_LAUNCH();
 }
 

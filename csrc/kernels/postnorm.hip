@@ -253,6 +253,36 @@ __global__ void __launch_bounds__(256) rmsnorm_cols_kernel(
   }
 }
 
+// The same for narrow parts (heads of at most 128 columns, n and all strides multiples of 4):
+// LPR lanes a part, 4 columns a lane, 256 / LPR parts a workgroup.
+template <typename S, int LPR>
+__global__ void __launch_bounds__(256) rmsnorm_heads_kernel(
+    S* __restrict__ out, const float* __restrict__ src, int lds, const S* __restrict__ w, int T,
+    int n, float eps, const float* __restrict__ gate, int ldg, int groups, int ldo,
+    float out_scale, bool silu) {
+  const long row = (long)blockIdx.x * (256 / LPR) + threadIdx.x / LPR;
+  if (row >= (long)T * groups) return;              // whole parts leave together
+  const int t = (int)(row / groups), go = (int)(row % groups) * n;
+  const int c = (threadIdx.x % LPR) * 4;
+  const bool on = c < n;
+  f32x4 v = {0.f, 0.f, 0.f, 0.f}, g = {0.f, 0.f, 0.f, 0.f};
+  if (on) {
+    v = *reinterpret_cast<const f32x4*>(src + (long)t * lds + go + c);
+    if (gate != nullptr) g = *reinterpret_cast<const f32x4*>(gate + (long)t * ldg + go + c);
+  }
+  float s = (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]);
+#pragma unroll
+  for (int o = LPR / 2; o > 0; o >>= 1) s += __shfl_xor(s, o, 64);
+  if (!on) return;
+  v *= 1.f / sqrtf(s / (float)n + eps);
+  if (w != nullptr) v *= ld4(w + go + c);
+  if (gate != nullptr) {
+#pragma unroll
+    for (int u = 0; u < 4; ++u) v[u] *= gate_of(g[u], silu);
+  }
+  st4(out + (long)t * ldo + go + c, v * out_scale);
+}
+
 // The same for few, wide rows (a decode step): one workgroup per row instead of one wave.
 template <typename S>
 __global__ void __launch_bounds__(256) rmsnorm_cols_block_kernel(
@@ -524,6 +554,18 @@ extern "C" int dli_rmsnorm_cols(void* out, const float* src, int lds, const void
   const int nb = (int)(((long)T * groups + 3) / 4);
   const bool vec4 = n % 4 == 0 && lds % 4 == 0 && ldg % 4 == 0 && ldo % 4 == 0 &&
                     (((uintptr_t)out | (uintptr_t)src | (uintptr_t)w | (uintptr_t)gate) & 15) == 0;
+  if (vec4 && n <= 128) {
+    const int lpr = n <= 32 ? 8 : n <= 64 ? 16 : 32;
+    const int nh = (int)(((long)T * groups + 256 / lpr - 1) / (256 / lpr));
+#define RH_LAUNCH(S, L)                                                                        \
+  rmsnorm_heads_kernel<S, L><<<nh, 256, 0, st>>>((S*)out, src, lds, (const S*)w, T, n, eps,     \
+                                                 gate, ldg, groups, ldo, out_scale, silu != 0)
+    if (lpr == 8) DT_SWITCH(dt, RH_LAUNCH(u16, 8), RH_LAUNCH(float, 8));
+    else if (lpr == 16) DT_SWITCH(dt, RH_LAUNCH(u16, 16), RH_LAUNCH(float, 16));
+    else DT_SWITCH(dt, RH_LAUNCH(u16, 32), RH_LAUNCH(float, 32));
+#undef RH_LAUNCH
+    DLI_RETURN_LAUNCH();
+  }
   DT_SWITCH(dt,
             (rmsnorm_cols_kernel<u16><<<nb, 256, 0, st>>>((u16*)out, src, lds, (const u16*)w, T,
                                                           n, eps, vec4, gate, ldg, groups, ldo,

@@ -64,6 +64,8 @@ class HybridLM(TransformerLM):
         if any(s.bias for s in cfg.layer_specs) and (cfg.residual_mult != 1.0 or cfg.streams
                                                      or cfg.post_norm):
             raise ValueError("output biases ride on the plain residual add (multiplier 1)")
+        if cfg.streams and cfg.loop and (cfg.loop_entry or cfg.loop_add):
+            raise ValueError("a loop that re-reads the embedding runs on the plain residual")
         for i, spec in enumerate(cfg.layer_specs):
             prepare_feed_forward(spec, params, f"layers.{i}.")
         super().__init__(cfg, params, 0, None, device)
@@ -126,9 +128,13 @@ class HybridLM(TransformerLM):
                 prev = H.prev_tokens(b.input_ids, kv_caches.prev_token, step.state_slots,
                                      step.cu_seqlens, step.max_seqlen, step.positions)
             return H.embedding_bigram(b.input_ids, prev, p["embed"], p.get("bigram"), *bg)
-        return H.embedding_f32(b.input_ids, p["embed"], scale=cfg.embed_scale,
-                               pos_table=p.get("pos_embed") if cfg.learned_pos else None,
-                               positions=b.positions)[0]
+        # (x, the copy x0 that the loop's passes read): one launch; x alone without such a loop
+        x, x0 = H.embedding_f32(b.input_ids, p["embed"],
+                                copy=bool(cfg.loop and (cfg.loop_entry or cfg.loop_add)),
+                                scale=cfg.embed_scale,
+                                pos_table=p.get("pos_embed") if cfg.learned_pos else None,
+                                positions=b.positions)
+        return x if x0 is None else (x, x0)
 
     def _postnorm_layers(self, xs, b: DeviceBatch, kv_caches) -> torch.Tensor:
         """Post-norm layers: every sublayer reads the stream itself and the norm follows the
@@ -173,7 +179,7 @@ class HybridLM(TransformerLM):
                 y = prev = None
         return H.hyper_mix(xs, y, prev, self._sum_streams, None)
 
-    def forward_layers(self, x: torch.Tensor, b: DeviceBatch, kv_caches) -> torch.Tensor:
+    def forward_layers(self, x, b: DeviceBatch, kv_caches) -> torch.Tensor:
         cfg, p = self.cfg, self.params
         if cfg.post_norm:
             return self._postnorm_layers(x, b, kv_caches)
@@ -182,7 +188,7 @@ class HybridLM(TransformerLM):
         eps, groups, m, off = cfg.norm_eps, cfg.norm_groups, cfg.residual_mult, cfg.norm_offset
         step = self._step_view(b, kv_caches.block_size)
         entries = kv_caches.entries
-        x0 = x.clone() if cfg.loop and (cfg.loop_entry or cfg.loop_add) else None
+        x, x0 = x if isinstance(x, tuple) else (x, None)
         pending = bias = None               # a sub-block's fp32 output (and bias) awaiting its add
         for ri, (li, t, first) in enumerate(self.runs):
             spec, lp = cfg.layer_specs[li], self.layers[li]
