@@ -162,7 +162,7 @@ ATTENTIONS = {
     "window_one": attention(2, 1, 8, size=1, keep=0),
     "all_kept": attention(2, 1, 8, size=4, keep=100),
     "matrix_core_32": attention(4, 2, 32, scale=0.2, rot_=rot(16, 900.0), size=13, keep=4),
-    "matrix_core_64": attention(4, 1, 64, scale=0.13, rot_=rot(64, 900.0), size=40, keep=2),
+    "matrix_core_64": attention(4, 1, 64, scale=0.13, rot_=rot(64, 900.0), size=37, keep=2),
     "matrix_core_128": attention(4, 2, 128, scale=0.09, rot_=rot(64, 900.0), size=30, keep=6)}
 
 
@@ -639,7 +639,7 @@ def test_registry_model_random_init_generates():
 @pytest.mark.parametrize("width,lay,n", [
     (128, retention(2, 64, 128, [0.97, 0.999], rot(32), dense(192)), 150),
     (192, retention(2, 128, 64, [0.9, 1.0], rot(128, 5000.0), dense(128)), 201),
-    (128, attention(4, 2, 64, 0.13, rot(32, 800.0), 40, 4, dense(256)), 333),
+    (128, attention(6, 2, 64, 0.11, rot(48, 800.0), 53, 4, dense(256)), 333),
     (192, attention(8, 2, 128, 0.09, rot(128, 3000.0), 100, 5, dense(64)), 410),
     (64, attention(16, 1, 128, 0.09, rot(64, 3000.0), 300, 1), 700)],
     ids=["retention_64", "retention_128", "attention_64", "attention_128", "attention_16_heads"])
