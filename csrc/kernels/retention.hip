@@ -442,7 +442,6 @@ int launch_step(const RetentionArgs& a, int num_seqs, hipStream_t st) {
   dim3 grid(a.H, num_seqs);
   if (R <= 1) retention_step_kernel<1><<<grid, 256, sh, st>>>(a, lg);
   else if (R <= 4) retention_step_kernel<4><<<grid, 256, sh, st>>>(a, lg);
-  else if (R <= 8) retention_step_kernel<8><<<grid, 256, sh, st>>>(a, lg);
   else if (R <= 16) retention_step_kernel<16><<<grid, 256, sh, st>>>(a, lg);
   else retention_step_kernel<32><<<grid, 256, sh, st>>>(a, lg);
   DLI_RETURN_LAUNCH();
