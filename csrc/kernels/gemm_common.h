@@ -20,9 +20,11 @@ enum { EPI_BF16 = 0, EPI_F32 = 1, EPI_SILU = 2, EPI_BIAS_GELU = 3, EPI_BIAS = 4,
        EPI_GELU_ERF = 6,
        // g sigmoid(1.702 g) (u + 1) over the interleaved gate/up weight, g = min(gate, L), u =
        // clamp(up, -L, L); `bias` points to the fp32 constant L on the device
-       EPI_CLAMP = 7 };
+       EPI_CLAMP = 7,
+       // relu(gate) * up over the interleaved gate/up weight
+       EPI_RELU = 8 };
 // epilogues that pair a gate block with the up block beside it (output width N / 2)
-constexpr bool epi_pairs(int epi) { return epi == EPI_SILU || epi == EPI_CLAMP; }
+constexpr bool epi_pairs(int epi) { return epi == EPI_SILU || epi == EPI_CLAMP || epi == EPI_RELU; }
 
 typedef __attribute__((address_space(3))) void lds_void;
 typedef const __attribute__((address_space(1))) void gbl_void;
@@ -207,7 +209,8 @@ __device__ __forceinline__ float clamp_swish_f(float g, float u, float lim) {
   return g / (1.f + __expf(-1.702f * g)) * (u + 1.f);
 }
 template <int EPI> __device__ __forceinline__ float pair_f(float g, float u, float lim) {
-  return EPI == EPI_CLAMP ? clamp_swish_f(g, u, lim) : silu_f(g) * u;
+  return EPI == EPI_CLAMP ? clamp_swish_f(g, u, lim)
+                          : EPI == EPI_RELU ? fmaxf(g, 0.f) * u : silu_f(g) * u;
 }
 // the constant of a pairing epilogue
 template <int EPI> __device__ __forceinline__ float pair_const(const u16* bias) {
@@ -316,6 +319,7 @@ int gemm_4w_set_slab_store(int mode);
 // an fp16 slab store (tiles, 8-phase) take DLI_EPI_SWITCH_S16
 #define DLI_EPI_SWITCH_S16(FN)                                                     \
   if (epi == EPI_CLAMP) return FN<EPI_CLAMP>(tile_cfg, DLI_GEMM_PASS);             \
+  if (epi == EPI_RELU) return FN<EPI_RELU>(tile_cfg, DLI_GEMM_PASS);               \
   if (epi == EPI_SLAB16) {                                                         \
     if (C != nullptr || splits < 2) return (int)hipErrorInvalidValue;              \
     return FN<EPI_SLAB16>(tile_cfg, DLI_GEMM_PASS);                                \

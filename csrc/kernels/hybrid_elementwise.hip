@@ -244,6 +244,7 @@ __device__ __forceinline__ float act_pair(int kind, float g, float u, float limi
     u = fminf(fmaxf(u, -limit), limit);
     return g / (1.f + expf(-1.702f * g)) * (u + 1.f);
   }
+  if (kind == 6) return fmaxf(g, 0.f) * u;
   if (kind == 0) return gelu_tanh32(g) * u;
   if (kind == 1) return g / (1.f + expf(-g)) * u;
   if (kind == 3) return 0.5f * g * (1.f + erff(g * 0.7071067811865476f));
@@ -253,7 +254,8 @@ __device__ __forceinline__ float act_pair(int kind, float g, float u, float limi
 
 // kind 0: gelu_tanh(gu[:, c]) * gu[:, F + c]; 1: silu(..) * ..; 2: gelu_tanh(gu[:, c]);
 // 3: the exact (erf) GELU of gu[:, c]; 4: gu[:, c] itself (a rounding copy of a column slice);
-// 5: g sigmoid(1.702 g) (u + 1) with g = min(gu[:, c], limit), u = clamp(gu[:, F + c], +-limit).
+// 5: g sigmoid(1.702 g) (u + 1) with g = min(gu[:, c], limit), u = clamp(gu[:, F + c], +-limit);
+// 6: relu(gu[:, c]) * gu[:, F + c].
 // nrows (nullable, device): rows from *nrows on hold no data and are skipped.
 // I: the projection's type (fp32, or bf16 bits when a tuned GEMM wrote it).
 template <typename I> __device__ __forceinline__ f32x4 ldin4(const I* p);
@@ -276,7 +278,7 @@ __global__ void __launch_bounds__(256) act_mul_kernel(
   if (nrows != nullptr && t >= *nrows) return;
   const I* r = gu + (long)t * ldg;
   stf(out + (long)t * ldo + c,
-      act_pair(kind, ldf(r + c), (kind >= 2 && kind != 5) ? 0.f : ldf(r + F + c), limit));
+      act_pair(kind, ldf(r + c), (kind >= 2 && kind < 5) ? 0.f : ldf(r + F + c), limit));
 }
 
 // 4 features a thread (F, ldg multiples of 4, 16-byte aligned rows): 16-byte loads
@@ -292,7 +294,7 @@ __global__ void __launch_bounds__(256) act_mul4_kernel(
   const I* r = gu + (long)t * ldg;
   const f32x4 g = ldin4(r + c);
   f32x4 u = f32x4{0.f, 0.f, 0.f, 0.f};
-  if (kind < 2 || kind == 5) u = ldin4(r + F + c);
+  if (kind < 2 || kind >= 5) u = ldin4(r + F + c);
 #pragma unroll
   for (int i = 0; i < 4; ++i)
     stf(out + (long)t * ldo + c + i, act_pair(kind, g[i], u[i], limit));
@@ -530,7 +532,7 @@ extern "C" int dli_token_shift(const float* h, const void* mu, float* state, con
 extern "C" int dli_act_mul(void* out, int ldo, const void* gu, int ldg, int T, int F, int kind,
                            const int* nrows, float limit, int in_dt, int dt, hipStream_t st) {
   if (T <= 0) return 0;
-  if (kind < 0 || kind > 5 || in_dt < 0 || in_dt > 1 || (in_dt == 0 && dt != 0))
+  if (kind < 0 || kind > 6 || in_dt < 0 || in_dt > 1 || (in_dt == 0 && dt != 0))
     return (int)hipErrorInvalidValue;
   const bool v4 = F % 4 == 0 && ldg % 4 == 0 && (uintptr_t)gu % 16 == 0;
   const int nb = (int)(((long)T * (v4 ? F / 4 : F) + 255) / 256);

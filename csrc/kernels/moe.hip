@@ -426,23 +426,16 @@ template <> __device__ __forceinline__ float rld<float>(const float* p) { return
 
 constexpr int ROUTER_MAX = 1024;
 
+// fp32 logits z[e] = W[e] . row, e < n, of the token row in LDS: waves take router rows in turn
 template <typename S>
-__global__ void __launch_bounds__(256) score_router_kernel(
-    float* __restrict__ topk_w, int* __restrict__ topk_ids, float* __restrict__ gates,
-    const S* __restrict__ h, int ldh, const S* __restrict__ W, const float* __restrict__ corr,
-    int D, int n, int n_gate, int top, bool vec, int groups, int keep, float wscale) {
-  extern __shared__ __attribute__((aligned(16))) float rsm[];                      // [D] row, [n + n_gate] logits
-  float* row = rsm;
-  float* z = rsm + D;
-  const int t = blockIdx.x;
+__device__ __forceinline__ void router_logits(const float* row, const S* __restrict__ W, float* z,
+                                              int D, int n, bool vec) {
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, nw = blockDim.x >> 6;
-  for (int c = threadIdx.x; c < D; c += blockDim.x) row[c] = rld(h + (long)t * ldh + c);
-  __syncthreads();
   if (vec) {
     // 16-byte loads of the router rows, 4 in flight a lane (D a multiple of the chunk)
     constexpr int CH = 16 / sizeof(S);
     const int nch = D / CH;
-    for (int e = wid; e < n + n_gate; e += nw) {
+    for (int e = wid; e < n; e += nw) {
       const S* wr = W + (long)e * D;
       float acc = 0.f;
       for (int c0 = lane; c0 < nch; c0 += 256) {
@@ -470,7 +463,7 @@ __global__ void __launch_bounds__(256) score_router_kernel(
       if (lane == 0) z[e] = acc;
     }
   } else {
-    for (int e = wid; e < n + n_gate; e += nw) {
+    for (int e = wid; e < n; e += nw) {
       const S* wr = W + (long)e * D;
       float acc = 0.f;
       for (int c = lane; c < D; c += 64) acc += row[c] * rld(wr + c);
@@ -478,6 +471,20 @@ __global__ void __launch_bounds__(256) score_router_kernel(
       if (lane == 0) z[e] = acc;
     }
   }
+}
+
+template <typename S>
+__global__ void __launch_bounds__(256) score_router_kernel(
+    float* __restrict__ topk_w, int* __restrict__ topk_ids, float* __restrict__ gates,
+    const S* __restrict__ h, int ldh, const S* __restrict__ W, const float* __restrict__ corr,
+    int D, int n, int n_gate, int top, bool vec, int groups, int keep, float wscale) {
+  extern __shared__ __attribute__((aligned(16))) float rsm[];                      // [D] row, [n + n_gate] logits
+  float* row = rsm;
+  float* z = rsm + D;
+  const int t = blockIdx.x;
+  for (int c = threadIdx.x; c < D; c += blockDim.x) row[c] = rld(h + (long)t * ldh + c);
+  __syncthreads();
+  router_logits(row, W, z, D, n + n_gate, vec);
   __syncthreads();
   if (threadIdx.x != 0) return;
   float m = -INFINITY;
@@ -520,6 +527,77 @@ __global__ void __launch_bounds__(256) score_router_kernel(
     topk_ids[(long)t * top + j] = best;
     topk_w[(long)t * top + j] = bz * inv * wscale;
     if (z[best] != -2.f) z[best] = -2.f;
+  }
+}
+
+// Router with sigmoid scores (sigmoid_router): the `top` largest fp32 logits (lowest index on ties),
+// weights sigmoid(logit). One workgroup per token, its first wave selects. A row of NaNs
+// still selects valid ids.
+template <typename S>
+__global__ void __launch_bounds__(256) sigmoid_router_kernel(
+    float* __restrict__ topk_w, int* __restrict__ topk_ids, const S* __restrict__ h, int ldh,
+    const S* __restrict__ W, int D, int n, int top, bool vec) {
+  extern __shared__ __attribute__((aligned(16))) float rsm[];                      // [D] row, [n] logits
+  float* row = rsm;
+  float* z = rsm + ((D + 3) & ~3);
+  const int t = blockIdx.x;
+  for (int c = threadIdx.x; c < D; c += blockDim.x) row[c] = rld(h + (long)t * ldh + c);
+  __syncthreads();
+  router_logits(row, W, z, D, n, vec);
+  __syncthreads();
+  if (threadIdx.x >= 64) return;
+  const int lane = threadIdx.x;
+  unsigned taken = 0;                              // of this lane's experts lane + 64 i (n <= 1024)
+  for (int j = 0; j < top; ++j) {
+    float bv = -INFINITY;
+    int bi = ROUTER_MAX;                           // none left
+    for (int i = 0; lane + 64 * i < n; ++i) {
+      const float v = z[lane + 64 * i];
+      if (!((taken >> i) & 1) && (bi == ROUTER_MAX || v > bv)) { bv = v; bi = lane + 64 * i; }
+    }
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) {
+      const float ov = __shfl_xor(bv, o, 64);
+      const int oi = __shfl_xor(bi, o, 64);
+      if (oi < ROUTER_MAX && (bi == ROUTER_MAX || ov > bv || (!(bv > ov) && oi < bi))) { bv = ov; bi = oi; }
+    }
+    bi = min(__shfl(bi, 0, 64), n - 1);
+    if (lane == (bi & 63)) taken |= 1u << (bi >> 6);
+    if (lane == 0) {
+      topk_ids[(long)t * top + j] = bi;
+      topk_w[(long)t * top + j] = 1.f / (1.f + expf(-z[bi]));
+    }
+  }
+}
+
+// Rows of routed experts whose weight multiplies their input: out[pos[i]] = w[i] * x[i / k]
+template <typename S>
+__global__ void __launch_bounds__(256) moe_scatter_weighed_kernel(
+    S* __restrict__ out, const S* __restrict__ x, int ldx, const float* __restrict__ w,
+    const int* __restrict__ pos, int n, int k, int dim, bool vec) {
+  constexpr int CH = 16 / sizeof(S);
+  const int units = vec ? dim / CH : dim;
+  const long gid = (long)blockIdx.x * blockDim.x + threadIdx.x;
+  if (gid >= (long)n * units) return;
+  const int i = (int)(gid / units), u = (int)(gid - (long)i * units);
+  const int p = pos[i];
+  if (p < 0) return;
+  const float f = w[i];
+  const S* src = x + (long)(i / k) * ldx;
+  S* dst = out + (long)p * dim;
+  if (!vec) {
+    if constexpr (sizeof(S) == 2) dst[u] = f2bf(f * bf2f(src[u]));
+    else dst[u] = f * src[u];
+    return;
+  }
+  if constexpr (sizeof(S) == 2) {
+    float v[8];
+    load8(src + u * 8, v);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) v[e] *= f;
+    store8(dst + u * 8, v);
+  } else {
+    *reinterpret_cast<f32x4*>(dst + u * 4) = f * *reinterpret_cast<const f32x4*>(src + u * 4);
   }
 }
 
@@ -591,5 +669,39 @@ extern "C" int dli_moe_combine_f32(float* out, const float* y, const void* route
                                                       (const float*)x, ldx, ys, gate, ldg, T, k,
                                                       dim, n_real);
   else return (int)hipErrorInvalidValue;
+  DLI_RETURN_LAUNCH();
+}
+
+extern "C" int dli_sigmoid_router(float* topk_w, int* topk_ids, const void* h, int ldh, const void* W,
+                                  int T, int D, int n, int top, int dt, hipStream_t st) {
+  if (T <= 0) return 0;
+  const size_t sh = ((size_t)((D + 3) & ~3) + n) * 4;
+  if (n < 1 || top < 1 || top > n || n > ROUTER_MAX || sh > 60000 || (dt != 0 && dt != 1))
+    return (int)hipErrorInvalidValue;
+  const bool vec = (uintptr_t)W % 16 == 0 && D % (dt == 0 ? 8 : 4) == 0;
+  if (dt == 0)
+    sigmoid_router_kernel<u16><<<T, 256, sh, st>>>(topk_w, topk_ids, (const u16*)h, ldh,
+                                                   (const u16*)W, D, n, top, vec);
+  else
+    sigmoid_router_kernel<float><<<T, 256, sh, st>>>(topk_w, topk_ids, (const float*)h, ldh,
+                                                     (const float*)W, D, n, top, vec);
+  DLI_RETURN_LAUNCH();
+}
+
+extern "C" int dli_moe_scatter_weighed(void* out, const void* x, int ldx, const float* w,
+                                       const int* pos, int n, int k, int dim, int dt,
+                                       hipStream_t st) {
+  if (n <= 0) return 0;
+  if (k < 1 || n % k || dim < 1 || (dt != 0 && dt != 1)) return (int)hipErrorInvalidValue;
+  const int CH = dt == 0 ? 8 : 4;
+  const bool vec = dim % CH == 0 && ldx % CH == 0 && ((uintptr_t)out | (uintptr_t)x) % 16 == 0;
+  const long total = (long)n * (vec ? dim / CH : dim);
+  const int nb = (int)((total + 255) / 256);
+  if (dt == 0)
+    moe_scatter_weighed_kernel<u16><<<nb, 256, 0, st>>>((u16*)out, (const u16*)x, ldx, w, pos, n, k,
+                                                        dim, vec);
+  else
+    moe_scatter_weighed_kernel<float><<<nb, 256, 0, st>>>((float*)out, (const float*)x, ldx, w, pos,
+                                                          n, k, dim, vec);
   DLI_RETURN_LAUNCH();
 }

@@ -19,6 +19,9 @@
 //   (dimension i with i + rot/2, by the step's table of cosines | sines), k times d^(-1/2); o_t
 //   is divided by its RMS per head and multiplied by silu(gate_t) -> S. Portions of more than
 //   a few tokens run the chunk form of retention.hip instead.
+// FORM 3, state-space recurrence: a_t = exp(-rate_h s_t), b_t = s_t = softplus(dt_t + dt_bias_h),
+//   and row t holds [H*dv v | G*d k | G*d q] (head h reads group h / (H/G)); o_t + skip_h v_t leaves
+//   in fp32. The sizes that the chunk form of ssd.hip does not take.
 //
 // Projection row of a token (fp32): [H*d q | H*d k | H*dv v | H*dv gate | H zi | H zf] (FORM 0
 // reads q, k, v only, FORM 2 also the gate). State: [slots, H, d, dv]; FORM 1 also nstate [slots, H, d + 1] = n, then
@@ -66,7 +69,13 @@ struct ScalarRecArgs {
   int H, d, dv, cw;               // cw: state columns per workgroup
   int ldd;                        // stride of decays (FORM 2 reads a table of powers)
   const float* table; int rot;    // FORM 2: [T, rot] cosines | sines
+  const float* dt; int ldt;       // FORM 3: [T, H]
+  const float* dt_bias; const float* rate; const float* skip; int G;
 };
+
+__device__ __forceinline__ float softplus32(float z) {
+  return z > 0.f ? z + log1pf(expf(-z)) : log1pf(expf(z));
+}
 
 template <typename S, int D, int P, int FORM>
 __global__ void __launch_bounds__(1024) scalar_recurrence_kernel(ScalarRecArgs a) {
@@ -92,11 +101,12 @@ __global__ void __launch_bounds__(1024) scalar_recurrence_kernel(ScalarRecArgs a
   const int slot = a.slots[s];
   const int t0 = a.cu[s], t1 = a.cu[s + 1];
   const int c = threadIdx.x % dvp, part = threadIdx.x / dvp;
-  const bool fused_norm = FORM != 0 && a.raw == nullptr;
+  constexpr bool PLAIN_OUT = FORM == 0 || FORM == 3;
+  const bool fused_norm = !PLAIN_OUT && a.raw == nullptr;
   if (slot < 0) {
     for (int t = t0; t < t1; ++t)
       if (c < ncol && part == 0) {
-        if (FORM == 0) ((float*)a.out)[(long)t * a.ldo + h * dv + c0 + c] = 0.f;
+        if (PLAIN_OUT) ((float*)a.out)[(long)t * a.ldo + h * dv + c0 + c] = 0.f;
         else if (fused_norm) stf((S*)a.out + (long)t * a.ldo + h * dv + c0 + c, 0.f);
         else a.raw[(long)t * H * dv + h * dv + c0 + c] = 0.f;
       }
@@ -123,7 +133,7 @@ __global__ void __launch_bounds__(1024) scalar_recurrence_kernel(ScalarRecArgs a
   const float qscale = FORM == 1 ? 1.f / sqrtf((float)d) : 1.f;
   const float kscale = FORM == 2 ? 1.f / sqrtf((float)d) : 1.f;
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, nw = blockDim.x >> 6;
-  const int voff = 2 * H * d + h * dv + c0, goff = 2 * H * d + H * dv + h * dv + c0;
+  const int voff = (FORM == 3 ? 0 : 2 * H * d) + h * dv + c0, goff = 2 * H * d + H * dv + h * dv + c0;
   const int ioff = 2 * H * d + 2 * H * dv + h, foff = ioff + H;
   for (int tc = t0; tc < t1; tc += TC) {
     const int n = min(TC, t1 - tc);
@@ -140,8 +150,9 @@ __global__ void __launch_bounds__(1024) scalar_recurrence_kernel(ScalarRecArgs a
     }
     const int dd = D ? D : d;
     for (int i = threadIdx.x; i < n * dd; i += blockDim.x) {
-      const float* row = a.proj + (long)(tc + i / dd) * a.ldp + h * dd + i % dd;
-      float q = row[0], k = row[H * dd];
+      const int q0 = FORM == 3 ? H * dv + (a.G + h / (H / a.G)) * dd : h * dd;
+      const float* row = a.proj + (long)(tc + i / dd) * a.ldp + q0 + i % dd;
+      float q = row[0], k = row[FORM == 3 ? -a.G * dd : H * dd];
       if (FORM == 2) {
         const int c2 = i % dd, hr = a.rot >> 1;
         if (c2 < a.rot) {
@@ -157,7 +168,13 @@ __global__ void __launch_bounds__(1024) scalar_recurrence_kernel(ScalarRecArgs a
       qv[i] = FORM == 0 ? silu32(q) : q * qscale;
       kv[i] = FORM == 0 ? silu32(k) : k;
     }
-    if (FORM != 1) {
+    if (FORM == 3) {
+      if (threadIdx.x < n) {
+        const float st = softplus32(a.dt[(long)(tc + threadIdx.x) * a.ldt + h] + a.dt_bias[h]);
+        ab[2 * threadIdx.x] = expf(-a.rate[h] * st);
+        ab[2 * threadIdx.x + 1] = st;
+      }
+    } else if (FORM != 1) {
       if (threadIdx.x < n) { ab[2 * threadIdx.x] = a.decays[(long)h * a.ldd]; ab[2 * threadIdx.x + 1] = 1.f; }
     } else {
       if (threadIdx.x < n) {                   // the gates' logarithms, a token a thread
@@ -248,11 +265,12 @@ __global__ void __launch_bounds__(1024) scalar_recurrence_kernel(ScalarRecArgs a
     __syncthreads();
     for (int tt = wid; tt < n; tt += nw) {
       const long t = tc + tt;
-      if (FORM == 0) {
+      if (PLAIN_OUT) {
         for (int k = lane; k < ncol; k += 64) {
           float o = ov[tt * dvp + k];
 #pragma unroll
           for (int pp = 1; pp < P; ++pp) o += ov[(pp * TC + tt) * dvp + k];
+          if (FORM == 3) o += a.skip[h] * vv[tt * dvp + k];
           ((float*)a.out)[t * a.ldo + h * dv + c0 + k] = o;
         }
       } else {
@@ -350,7 +368,8 @@ extern "C" int dli_scalar_recurrence(const float* proj, int ldp, int form, const
     return (int)hipErrorInvalidValue;
   if (cw == 0 || cw >= dv) { cw = dv; raw = form == 1 ? nullptr : raw; }
   ScalarRecArgs a{proj, ldp, decays, if_b, cap, norm_w, eps, state, nstate, slots, cu, positions,
-                  out, ldo, out_scale, raw, H, d, dv, cw, 1, nullptr, 0};
+                  out, ldo, out_scale, raw, H, d, dv, cw, 1, nullptr, 0, nullptr, 0, nullptr, nullptr,
+                  nullptr, 1};
   if (form == 0) {
     if (decays == nullptr || out == nullptr) return (int)hipErrorInvalidValue;
     return launch_scalar_recurrence<float, 0>(a, num_seqs, st);
@@ -370,7 +389,24 @@ int retention_walk(const float* proj, int ldp, const float* table, int rot, cons
                    const int* positions, void* out, int ldo, int num_seqs, int H, int d, int dv,
                    int cw, float* raw, int dt, hipStream_t st) {
   ScalarRecArgs a{proj, ldp, decay_pow + 1, nullptr, 0.f, nullptr, eps, state, nullptr, slots, cu,
-                  positions, out, ldo, 1.f, raw, H, d, dv, cw, ldd, table, rot};
+                  positions, out, ldo, 1.f, raw, H, d, dv, cw, ldd, table, rot, nullptr,
+                  0, nullptr, nullptr, nullptr, 1};
   if (dt == 0) return launch_scalar_recurrence<u16, 2>(a, num_seqs, st);
   return launch_scalar_recurrence<float, 2>(a, num_seqs, st);
+}
+
+// the walk form of the state-space recurrence (see ssd.hip, which takes most sizes): xc [T, ldx] fp32
+// filtered rows, y [T, H*P] fp32, column blocks of cw (0: one block)
+extern "C" int dli_ssd_walk(const float* xc, int ldx, const float* dts, int ldt, const float* dt_bias,
+                            const float* rate, const float* skip, float* state, const int* slots,
+                            const int* cu, const int* positions, float* y, int num_seqs,
+                            int max_seqlen, int H, int N, int P, int G, int cw, hipStream_t st) {
+  if (num_seqs <= 0 || max_seqlen <= 0) return 0;
+  if (H < 1 || G < 1 || H % G || N < 1 || P < 1 || state == nullptr || slots == nullptr || cw < 0 ||
+      (cw > 0 && cw % 64) || num_seqs > 65535 || ldx < H * P + 2 * G * N)
+    return (int)hipErrorInvalidValue;
+  if (cw == 0 || cw >= P) cw = P;
+  ScalarRecArgs a{xc, ldx, nullptr, nullptr, 0.f, nullptr, 0.f, state, nullptr, slots, cu, positions,
+                  y, H * P, 1.f, nullptr, H, N, P, cw, 1, nullptr, 0, dts, ldt, dt_bias, rate, skip, G};
+  return launch_scalar_recurrence<float, 3>(a, num_seqs, st);
 }

@@ -5,8 +5,8 @@
 //                    per step and rotation: the angle is formed in double and rounded once
 //  * rope_prepare    q / k (/ v) of an attention with rotated queries and keys: bias, the
 //                    rotation of the first `rot` dims of every head (dimension i with i +
-//                    rot/2), rotated k and v -> cache rows, q -> S. tied: there is no v, the
-//                    value row is the key before its rotation.
+//                    rot/2, or 2i with 2i + 1), rotated k and v -> cache rows, q -> S. tied: there
+//                    is no v, the value row is the key before its rotation. G = 0: queries only.
 #include "common.h"
 
 namespace {
@@ -119,6 +119,76 @@ __global__ void __launch_bounds__(256) rope_prepare_kernel(
   }
 }
 
+// The same for adjacent pairs (2i, 2i + 1). A unit is 2 VEC columns of a rotated part (VEC pairs), or
+// 2 VEC columns that pass (the last unit of a head may be cut short: VEC = 1, odd widths).
+template <typename S, int VEC>
+__global__ void __launch_bounds__(256) rope_prepare_adjacent_kernel(
+    const float* __restrict__ proj, int ldp, const S* __restrict__ bias,
+    const float* __restrict__ table, int rot, int T, int H, int G, int d, int dv, int tied,
+    S* __restrict__ q_out, S* __restrict__ kcache, S* __restrict__ vcache,
+    const int* __restrict__ slots) {
+  constexpr int W = 2 * VEC;
+  const int up = (d + W - 1) / W, uv = (dv + W - 1) / W;
+  const int nu = (H + G) * up + (tied ? 0 : G * uv);
+  const long gid = (long)blockIdx.x * blockDim.x + threadIdx.x;
+  if (gid >= (long)T * nu) return;
+  const int t = (int)(gid / nu), u = (int)(gid - (long)t * nu);
+  const bool is_v = u >= (H + G) * up;
+  const int uu = is_v ? u - (H + G) * up : u, per = is_v ? uv : up, width = is_v ? dv : d;
+  const int h = uu / per, c = (uu - h * per) * W;
+  const bool is_q = !is_v && h < H;
+  const int slot = is_q ? 0 : slots[t];
+  if (slot < 0) return;
+  const int src = (is_v ? (H + G) * d : 0) + h * width + c;
+  const float* row = proj + (long)t * ldp + src;
+  const int n = min(W, width - c);
+  float v[W];
+  if constexpr (VEC == 2) {
+    const f32x4 x = *reinterpret_cast<const f32x4*>(row);
+    v[0] = x[0]; v[1] = x[1]; v[2] = x[2]; v[3] = x[3];
+  } else {
+    v[0] = row[0];
+    v[1] = n > 1 ? row[1] : 0.f;
+  }
+  if (bias != nullptr) {
+#pragma unroll
+    for (int i = 0; i < W; ++i)
+      if (i < n) v[i] += ldf(bias + src + i);
+  }
+  const auto put = [&](S* p) {
+    if constexpr (VEC == 2) {
+      if constexpr (sizeof(S) == 2) {
+        uint2 pk;
+        pk.x = pack2bf(v[0], v[1]);
+        pk.y = pack2bf(v[2], v[3]);
+        *reinterpret_cast<uint2*>(p) = pk;
+      } else {
+        *reinterpret_cast<f32x4*>(p) = f32x4{v[0], v[1], v[2], v[3]};
+      }
+    } else {
+      stf(p, v[0]);
+      if (n > 1) stf(p + 1, v[1]);
+    }
+  };
+  if (is_v) {
+    put(vcache + (long)slot * G * dv + h * dv + c);
+    return;
+  }
+  if (!is_q && tied && vcache != kcache) put(vcache + (long)slot * G * d + (src - H * d));
+  if (c < rot) {                                     // rot is even: whole pairs
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) {
+      const int k = (c >> 1) + i;
+      if (2 * k >= rot) continue;
+      const float cs = table[(long)t * rot + k], sn = table[(long)t * rot + (rot >> 1) + k];
+      const float a = v[2 * i], b = v[2 * i + 1];
+      v[2 * i] = a * cs - b * sn;
+      v[2 * i + 1] = b * cs + a * sn;
+    }
+  }
+  put(is_q ? q_out + (long)t * H * d + src : kcache + (long)slot * G * d + (src - H * d));
+}
+
 }  // namespace
 
 extern "C" int dli_rotation_table(float* out, const int* positions, const double* freq, int T,
@@ -131,14 +201,28 @@ extern "C" int dli_rotation_table(float* out, const int* positions, const double
 
 extern "C" int dli_rope_prepare(const float* proj, int ldp, const void* bias, const float* table,
                                 int rot, int T, int H, int G, int d, int dv, int tied,
-                                void* q_out, void* kcache, void* vcache, const int* slots, int dt,
+                                int adjacent, void* q_out, void* kcache, void* vcache, const int* slots, int dt,
                                 hipStream_t st) {
   if (T <= 0) return 0;
-  if (H < 1 || G < 1 || H % G || d < 1 || dv < 1 || rot < 0 || (rot & 1) || rot > d ||
+  if (H < 1 || G < 0 || (G > 0 && (H % G || kcache == nullptr || vcache == nullptr)) || d < 1 || dv < 1 || rot < 0 || (rot & 1) || rot > d ||
       (rot > 0 && table == nullptr) || (tied && dv != d) || (dt != 0 && dt != 1))
     return (int)hipErrorInvalidValue;
   const uintptr_t mis = (uintptr_t)proj | (uintptr_t)table | (uintptr_t)q_out |
                         (uintptr_t)kcache | (uintptr_t)vcache;
+  if (adjacent) {
+    const bool v4 = d % 4 == 0 && dv % 4 == 0 && ldp % 4 == 0 && mis % 16 == 0;
+    const int w = v4 ? 4 : 2;
+    const long tot = (long)T * ((H + G) * ((d + w - 1) / w) + (tied ? 0 : G * ((dv + w - 1) / w)));
+    const int blocks = (int)((tot + 255) / 256);
+#define RA_LAUNCH(S, VV)                                                                        \
+  rope_prepare_adjacent_kernel<S, VV><<<blocks, 256, 0, st>>>(                                  \
+      proj, ldp, (const S*)bias, table, rot, T, H, G, d, dv, tied, (S*)q_out, (S*)kcache,       \
+      (S*)vcache, slots)
+    if (v4) { if (dt == 0) RA_LAUNCH(u16, 2); else RA_LAUNCH(float, 2); }
+    else { if (dt == 0) RA_LAUNCH(u16, 1); else RA_LAUNCH(float, 1); }
+#undef RA_LAUNCH
+    DLI_RETURN_LAUNCH();
+  }
   const bool v4 = d % 4 == 0 && dv % 4 == 0 && rot % 8 == 0 && ldp % 4 == 0 && mis % 16 == 0;
   const int V = v4 ? 4 : 1;
   const int up = (rot / 2 + d - rot) / V;

@@ -107,6 +107,12 @@ class HybridCache:
                             normed, rotated keys and values; the memory side's matrix, and its
                             normaliser vector followed by its running maximum
 
+    * ``rope_attention`` with ``kv_from``: the tensors of that layer's run (it writes nothing)
+    * ``ssd``:              (state [state_slots, H, d, dv] fp32, conv [state_slots, taps,
+                            channels] fp32): row p mod taps of conv holds the convolution's
+                            input at position p
+    * ``side_by_side``:     the left mixer's tensors, then the right one's
+
     ``shift_states[run]`` is [state_slots, D] fp32 for a layer with token shift (the previous
     token's mixer input), else None. ``prev_token`` is int32 [state_slots] for a design whose
     embedding reads the previous token (hashed bigrams), else None.
@@ -136,6 +142,15 @@ class HybridCache:
                 self.entries.append(self.entries[run_of[s.kv_from]])
                 run_of[li] = ri
                 continue
+            if s.kind == "rope_attention" and s.kv_from >= 0:
+                self.entries.append(self.entries[run_of[s.kv_from]])
+                run_of[li] = ri
+                continue
+            if s.kind == "side_by_side":
+                self.entries.append(self._entry(s.left, rows, device, dtype)
+                                    + self._entry(s.right, rows, device, dtype))
+                run_of[li] = ri
+                continue
             if s.kind == "talk_attention":
                 if s.kv_from >= 0:
                     e = self.entries[run_of[s.kv_from]]
@@ -149,10 +164,8 @@ class HybridCache:
             if s.kind == "attention":
                 e = (torch.zeros(rows, s.kv_heads * s.dim, dtype=dtype, device=device),
                      torch.zeros(rows, s.kv_heads * s.dim, dtype=dtype, device=device))
-            elif s.kind == "rope_attention":
-                k = torch.zeros(rows, s.kv_heads * s.dim, dtype=dtype, device=device)
-                e = (k, k if s.tied_values and not s.rot_dims else
-                     torch.zeros(rows, s.kv_heads * s.vdim, dtype=dtype, device=device))
+            elif s.kind in ("rope_attention", "ssd"):
+                e = self._entry(s, rows, device, dtype)
             elif s.kind == "latent_attention":
                 e = (torch.zeros(rows, s.kv_rank + s.rot_dim, dtype=dtype, device=device),)
             elif s.kind == "parallel":
@@ -167,6 +180,16 @@ class HybridCache:
                 e = (torch.zeros(state_slots, s.heads, s.dim, s.vdim, dtype=torch.float32,
                                  device=device),)
             self.entries.append(e)
+
+    def _entry(self, s, rows: int, device, dtype) -> tuple:
+        """The tensors of one run of a mixer that can stand alone or beside another."""
+        if s.kind == "ssd":
+            n = self.state_slots
+            return (torch.zeros(n, s.heads, s.dim, s.vdim, dtype=torch.float32, device=device),
+                    torch.zeros(n, s.taps, s.conv_channels, dtype=torch.float32, device=device))
+        k = torch.zeros(rows, s.kv_heads * s.dim, dtype=dtype, device=device)
+        return (k, k if s.tied_values and not s.rot_dims else
+                torch.zeros(rows, s.kv_heads * s.vdim, dtype=dtype, device=device))
 
     def layers(self) -> "HybridCache":
         """What the runner hands to the model: the cache itself (entries + block size)."""

@@ -34,7 +34,17 @@ class LayerSpec:
     each head's read-out divided by its own RMS, SiLU output gate) and ``rope_attention``
     (grouped-query softmax attention over ``window`` positions plus the first ``keep_first``
     ones, the first ``rot_dims`` dims of q and k rotated; ``bias``: q / k / v / output
-    projections carry biases; ``tied_values``: the values are the keys before their rotation).
+    projections carry biases; ``tied_values``: the values are the keys before their rotation;
+    ``rot_adjacent``: rotated pairs are (2i, 2i+1) instead of (i, i + rot_dims/2);
+    ``rot_llama3``: frequencies scaled by wavelength; ``out_gate``: the concatenated heads are
+    multiplied by the sigmoid of a projection of the mixer input; ``kv_from``: keys and values
+    are another layer's cache rows).
+    ``ssd`` (state-space recurrence: a [dim, vdim] state per head with a decay and a step size
+    per token, the [dim] input and output vectors shared by the heads of one of ``groups``
+    groups, a causal convolution of ``taps`` taps per channel in front, a skip per head, a SiLU
+    gate and an RMS norm over ``norm_parts`` parts behind) and ``side_by_side`` (the mixers
+    ``left`` and ``right`` on the same input; each output RMS-normed with a weight of its own,
+    the mean of the two).
 
     feed-forward kinds (``ff_kind``): ``gated_gelu`` (down(gelu(gate) * up)), ``gelu``
     (down(gelu(up))) and ``moe`` (``experts`` gated-SiLU experts of width ``ff`` plus
@@ -42,10 +52,12 @@ class LayerSpec:
     correction and weighted by the un-renormalised score, and a shared expert of width
     ``shared_ff`` behind a per-token sigmoid gate), ``gated_silu`` (down(silu(gate) * up)) and
     ``clamp_swish`` (down(g sigmoid(1.702 g) (u + 1)), g = min(gate, ``act_limit``), u = up
-    clamped to +-``act_limit``).
+    clamped to +-``act_limit``) and ``gated_relu`` (down(relu(gate) * up)).
     A mixture with ``router`` = ``logit_topk`` picks the ``top`` largest biased logits and
     weighs them by the softmax over the chosen ones; ``expert_act`` = ``gelu_erf`` makes the
-    experts (and the shared one, then ungated) down(gelu(up)) with the exact GELU."""
+    experts (and the shared one, then ungated) down(gelu(up)) with the exact GELU. ``router`` =
+    ``sigmoid``: every expert's score is the sigmoid of its logit and weighs, un-renormalised,
+    what goes into a chosen expert (the sum over the experts' outputs is plain)."""
     kind: str
     heads: int
     dim: int
@@ -66,7 +78,8 @@ class LayerSpec:
     identity: int = 0
     top: int = 0
     shared_ff: int = 0
-    router: str = "score"     # "score" (softmax score + correction) | "logit_topk"
+    router: str = "score"     # "score" (softmax score + correction) | "logit_topk" |
+                              # "group_score" | "sigmoid" (weighs the experts' input)
     expert_act: str = "silu_mul"   # "silu_mul" (gated) | "gelu_erf" (ungated)
     q_rank: int = 0           # latent attention: width of the query latent (0: none)
     head_gate: bool = False   # latent attention: one sigmoid output gate per head
@@ -87,13 +100,25 @@ class LayerSpec:
     keep_first: int = 0       # rope_attention: these first positions stay visible past the window
     bias: bool = False        # rope_attention: biased projections
     tied_values: bool = False     # rope_attention: values = the keys before their rotation
+    rot_adjacent: bool = False    # rope_attention: rotated pairs (2i, 2i+1)
+    rot_llama3: tuple = ()    # rope_attention: (factor, low, high, original length) or ()
+    out_gate: bool = False    # rope_attention: elementwise sigmoid gate on the heads' output
+    taps: int = 0             # ssd: taps of the convolution (the last is the current token's)
+    groups: int = 1           # ssd: groups of heads that share input and output vectors
+    norm_parts: int = 1       # ssd: parts of the gated read-out that are normed by themselves
 
     @property
     def has_state(self) -> bool:
         """The layer keeps something per sequence besides cache rows: a recurrent state, or
         the previous token's mixer input."""
-        return self.kind in ("hgrn2", "gla", "lightning", "parallel", "mlstm",
-                             "retention") or self.shift
+        return self.kind in ("hgrn2", "gla", "lightning", "parallel", "mlstm", "retention",
+                             "ssd") or self.shift or (
+            self.kind == "side_by_side" and (self.left.has_state or self.right.has_state))
+
+    @property
+    def conv_channels(self) -> int:
+        """ssd: channels of the convolution, values | input vectors | output vectors."""
+        return self.heads * self.vdim + 2 * self.groups * self.dim
 
     @classmethod
     def from_dict(cls, d: dict) -> "LayerSpec":
@@ -101,7 +126,7 @@ class LayerSpec:
         for side in ("left", "right"):
             if isinstance(kw.get(side), dict):
                 kw[side] = cls.from_dict(kw[side])
-        for k in ("decays", "rot_scaling"):
+        for k in ("decays", "rot_scaling", "rot_llama3"):
             if k in kw:
                 kw[k] = tuple(kw[k] or ())
         return cls(**kw)
@@ -112,7 +137,7 @@ class ModelConfig:
     name: str
     arch: str                 # "llama" (llama / mixtral family), "gpt2", or a hybrid
                               # (layer-list) design: "buborax", "pulunex", "risutar",
-                              # "lapunex", "bamudra"
+                              # "lapunex", "bamudra", "lutovik"
     hidden_size: int
     num_layers: int
     num_heads: int
@@ -160,6 +185,8 @@ class ModelConfig:
     loop_entry: bool = True
     # every pass of the loop but the first starts with x = x + x0 (x0 = the embedding output)
     loop_add: bool = False
+    # a second norm follows every sublayer: x += norm_b(sublayer(norm(x)))
+    sandwich: bool = False
 
     @property
     def is_hybrid(self) -> bool:
@@ -242,13 +269,13 @@ class ModelConfig:
     def cache_row_width(self, layer: int) -> int:
         """Cached elements per token of one run of hybrid layer ``layer``."""
         s = self.layer_specs[layer]
+        if s.kind == "side_by_side":
+            s = s.left                              # the attention side's rows
         if s.kind == "attention":
             return 2 * s.kv_heads * s.dim           # normed keys + raw keys (the values)
         if s.kind == "latent_attention":
             return 0 if s.kv_from >= 0 else s.kv_rank + s.rot_dim
-        if s.kind == "rope_attention":
-            return s.kv_heads * (s.dim + s.vdim)
-        if s.kind == "talk_attention":
+        if s.kind in ("rope_attention", "talk_attention"):
             return 0 if s.kv_from >= 0 else s.kv_heads * (s.dim + s.vdim)
         if s.kind == "parallel":
             return s.left.kv_heads * (s.left.dim + s.left.vdim)
@@ -417,10 +444,31 @@ BAMUDRA_TINY = hybrid_config(
         replace(_BAMUDRA_RETENTION, ff=160, ff_kind="clamp_swish", act_limit=1.0)),
     loop=(1, 3, 2), norm_eps=1e-5, loop_entry=False, loop_add=True)
 
+# Lutovik at test size: attention beside a state-space recurrence, adjacent-pair rotation with
+# scaled frequencies, a layer on another layer's cache, norms before and after every sublayer,
+# a gated ReLU and routed feed-forwards whose scores weigh the experts' input
+_LUTOVIK_SIDES = dict(
+    left=LayerSpec("rope_attention", heads=4, kv_heads=2, dim=32, vdim=48, window=1 << 30,
+                   scale=0.18, rot_dims=16, rot_base=3000.0, out_gate=True),
+    right=LayerSpec("ssd", heads=6, dim=16, vdim=16, taps=3, groups=2, norm_parts=2))
+_LUTOVIK_ATTENTION = dict(heads=4, kv_heads=1, dim=32, vdim=32, window=1 << 30, scale=0.18,
+                          rot_dims=8, rot_base=1000.0, rot_adjacent=True,
+                          rot_llama3=(4.0, 1.0, 4.0, 256.0))
+_LUTOVIK_MOE = dict(ff_kind="moe", router="sigmoid", ff=48, experts=6, top=2, shared_ff=64)
+LUTOVIK_TINY = hybrid_config(
+    "lutovik-tiny", width=128, vocab=384, arch="lutovik",
+    layer_specs=(
+        LayerSpec("side_by_side", heads=4, kv_heads=2, dim=32, vdim=48, ff=160,
+                  ff_kind="gated_relu", **_LUTOVIK_SIDES),
+        LayerSpec("rope_attention", **_LUTOVIK_ATTENTION, **_LUTOVIK_MOE),
+        LayerSpec("rope_attention", **_LUTOVIK_ATTENTION, kv_from=1, **_LUTOVIK_MOE),
+        LayerSpec("side_by_side", heads=4, kv_heads=2, dim=32, vdim=48, ff=0, **_LUTOVIK_SIDES)),
+    norm_eps=1e-6, embed_scale=8.0, norm_offset=1.0, sandwich=True)
+
 _REGISTRY = {c.name: c for c in
              (GPT2, LLAMA3_8B, LLAMA3_70B, MIXTRAL_8X7B, LLAMA_TINY, LLAMA_TINY128,
               LLAMA_TINY8, MIXTRAL_TINY, MIXTRAL_TINY8E, GPT2_TINY, BUBORAX_TINY, PULUNEX_TINY,
-              RISUTAR_TINY, LAPUNEX_TINY, BAMUDRA_TINY)}
+              RISUTAR_TINY, LAPUNEX_TINY, BAMUDRA_TINY, LUTOVIK_TINY)}
 
 _ALIASES = {
     "openai-community/gpt2": "gpt2",

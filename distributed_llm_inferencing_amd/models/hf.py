@@ -25,8 +25,9 @@ from typing import Dict, Iterable, Iterator, Optional, Tuple
 import torch
 
 from .configs import ModelConfig
-from .weights import (from_bamudra_state_dict, from_buborax_state_dict, from_hf_state_dict, from_lapunex_state_dict,
-                      from_pulunex_state_dict, from_risutar_state_dict)
+from .weights import (from_bamudra_state_dict, from_buborax_state_dict, from_hf_state_dict,
+                      from_lapunex_state_dict, from_lutovik_state_dict, from_pulunex_state_dict,
+                      from_risutar_state_dict)
 
 
 def is_hf_dir(d) -> bool:
@@ -59,7 +60,7 @@ def find_hf_dir(root: str, name: str) -> Optional[Path]:
     return None
 
 
-NATIVE_ARCHS = ("Buborax", "Pulunex", "Risutar", "Lapunex", "Bamudra")
+NATIVE_ARCHS = ("Buborax", "Pulunex", "Risutar", "Lapunex", "Bamudra", "Lutovik")
 
 
 def buborax_config(c: dict, name: Optional[str] = None) -> ModelConfig:
@@ -351,10 +352,78 @@ def bamudra_config(c: dict, name: Optional[str] = None) -> ModelConfig:
                          loop_entry=False, loop_add=bool(loop))
 
 
+def lutovik_config(c: dict, name: Optional[str] = None) -> ModelConfig:
+    """A Lutovik ``config.json``: ``width``, ``vocab``, ``embedding`` {scale}, ``norm`` {eps} and
+    ``layers``, a list of {type, mixer, mlp}: type ``attention`` with mixer {heads, kv_heads, dim,
+    vdim, scale, rot {base, dims, scaling {factor, low, high, original}}, kv_from} or ``parallel``
+    with mixer {left: an attention's {heads, kv_heads, dim, vdim, scale, rot}, right: {heads,
+    vdim, state, groups, conv, norm_groups}}; mlp null, {kind: dense, ff} or {kind: moe, expert
+    {ff}, router {experts, top}, shared {ff} or null}. Every size and constant is read from it."""
+    from .configs import LayerSpec, hybrid_config
+
+    def attention(mx, where, **kw):
+        H, d = int(mx["heads"]), int(mx["dim"])
+        G = int(mx.get("kv_heads") or H)
+        if H < 1 or G < 1 or H % G:
+            raise ValueError(f"{where}: heads {H} must be a multiple of kv_heads {G}")
+        rot = mx.get("rot") or {}
+        dims = int(rot.get("dims") or 0)
+        if dims % 2 or dims > d:
+            raise ValueError(f"{where}: rot.dims {dims} of a head of {d}")
+        sc = rot.get("scaling") or {}
+        scaling = tuple(float(sc[k]) for k in ("factor", "low", "high", "original")) if sc else ()
+        return LayerSpec("rope_attention", heads=H, kv_heads=G, dim=d, vdim=int(mx.get("vdim", d)),
+                         window=1 << 30, scale=float(mx.get("scale", d ** -0.5)), rot_dims=dims,
+                         rot_base=float(rot.get("base", 10000.0)), rot_llama3=scaling, **kw)
+
+    specs = []
+    for i, L in enumerate(c["layers"]):
+        mx, kind, where = L["mixer"], L["type"], f"layer {i}"
+        mlp = L.get("mlp")
+        ff = dict(ff=0)
+        if mlp and mlp.get("kind") == "dense":
+            ff = dict(ff=int(mlp["ff"]), ff_kind="gated_relu")
+        elif mlp and mlp.get("kind") == "moe":
+            r, shared = mlp["router"], mlp.get("shared")
+            ff = dict(ff=int(mlp["expert"]["ff"]), ff_kind="moe", router="sigmoid",
+                      experts=int(r["experts"]), top=int(r["top"]),
+                      shared_ff=int(shared["ff"]) if shared else 0)
+            if not 1 <= ff["top"] <= ff["experts"]:
+                raise ValueError(f"{where}: {ff['top']} of {ff['experts']} experts")
+        elif mlp:
+            raise ValueError(f"unsupported feed-forward kind '{mlp.get('kind')}'")
+        if kind == "attention":
+            src = mx.get("kv_from")
+            s = attention(mx, where, rot_adjacent=True, kv_from=-1 if src is None else int(src), **ff)
+            if s.kv_from >= 0:
+                o = specs[s.kv_from] if s.kv_from < i else None
+                if (o is None or o.kind != "rope_attention" or o.kv_from >= 0
+                        or (o.kv_heads, o.dim, o.vdim) != (s.kv_heads, s.dim, s.vdim)):
+                    raise ValueError(f"{where}: layer {s.kv_from} has no keys and values of these sizes")
+            specs.append(s)
+        elif kind == "parallel":
+            left, r = attention(mx["left"], where, out_gate=True), mx["right"]
+            right = LayerSpec("ssd", heads=int(r["heads"]), dim=int(r["state"]), vdim=int(r["vdim"]),
+                              taps=int(r["conv"]), groups=int(r["groups"]),
+                              norm_parts=int(r["norm_groups"]))
+            if (right.heads % right.groups or right.taps < 1
+                    or right.heads * right.vdim % right.norm_parts):
+                raise ValueError(f"{where}: heads, groups and norm_groups do not divide")
+            specs.append(LayerSpec("side_by_side", heads=left.heads, kv_heads=left.kv_heads,
+                                   dim=left.dim, vdim=left.vdim, left=left, right=right, **ff))
+        else:
+            raise ValueError(f"unsupported mixer type '{kind}'")
+    return hybrid_config(name or c.get("_name_or_path") or "lutovik", int(c["width"]),
+                         int(c["vocab"]), specs,
+                         norm_eps=float((c.get("norm") or {}).get("eps", 1e-6)), arch="lutovik",
+                         embed_scale=float((c.get("embedding") or {}).get("scale", 1.0)),
+                         norm_offset=1.0, sandwich=True)
+
+
 def config_from_hf(c: dict, name: Optional[str] = None) -> ModelConfig:
     """Map a ``config.json``: HF llama / mistral / mixtral / gpt2 model types, or one of the
     native layer-list designs (``architecture``: Buborax, Pulunex, Risutar, Lapunex,
-    Bamudra)."""
+    Bamudra, Lutovik)."""
     if c.get("architecture") == "Buborax":
         return buborax_config(c, name)
     if c.get("architecture") == "Pulunex":
@@ -365,6 +434,8 @@ def config_from_hf(c: dict, name: Optional[str] = None) -> ModelConfig:
         return lapunex_config(c, name)
     if c.get("architecture") == "Bamudra":
         return bamudra_config(c, name)
+    if c.get("architecture") == "Lutovik":
+        return lutovik_config(c, name)
     mt = c.get("model_type", "")
     name = name or c.get("_name_or_path") or mt
     if mt == "gpt2":
@@ -482,6 +553,8 @@ def load_hf_dir(d, device="cpu", dtype=torch.bfloat16, name: Optional[str] = Non
             params = from_lapunex_state_dict(cfg, sd, dtype=dtype)
         elif cfg.arch == "bamudra":
             params = from_bamudra_state_dict(cfg, sd, dtype=dtype)
+        elif cfg.arch == "lutovik":
+            params = from_lutovik_state_dict(cfg, sd, dtype=dtype)
         elif cfg.is_hybrid:
             params = from_buborax_state_dict(cfg, sd, dtype=dtype)
         else:

@@ -1,7 +1,7 @@
-"""Hybrid decoder (archs ``buborax``, ``pulunex``, ``risutar``, ``lapunex``, ``bamudra``): a
-layer list that mixes windowed attention, latent attention, gated linear recurrences (HGRN2,
+"""Hybrid decoder (archs ``buborax``, ``pulunex``, ``risutar``, ``lapunex``, ``bamudra``,
+``lutovik``): a layer list that mixes windowed attention, latent attention, gated linear recurrences (HGRN2,
 gated linear attention, fixed-decay linear attention with or without rotation, a matrix memory
-beside a sink attention) and block attention with head-mixed scores; dense, gated and routed feed-forwards; a shared-weight loop,
+beside a sink attention, a state-space recurrence beside a gated attention) and block attention with head-mixed scores; dense, gated and routed feed-forwards; a shared-weight loop,
 grouped RMS norms, token shift and an fp32 residual stream (or several hyper-connected
 streams) — served by the same engine, scheduler, block manager and runner as the transformer
 families.
@@ -26,6 +26,14 @@ and stream mix M runs
 
 and the final norm reads the sum of the streams (``ops.hybrid.hyper_mix`` fuses a sublayer's
 write-back with the next sublayer's read and norm).
+
+Sandwich-norm designs (``cfg.sandwich``; ``lutovik``) run
+
+    per layer: x += norm_b(mixer(norm(x)));  x += norm_b(ff(norm(x)))
+
+where one launch norms a sublayer's output, adds it and leaves the next sublayer's normed input
+(``ops.hybrid.sandwich_add``), also when that output is the mean of two mixers' normed outputs or
+the sum of a token's routed experts.
 
 * Layers [start, stop) of the loop run ``times`` times with the same weights; a pass starts
   with x = W_in [x ; x0] + step[pass] (x0 = the embedding output), or every pass but the first
@@ -64,6 +72,10 @@ class HybridLM(TransformerLM):
         if any(s.bias for s in cfg.layer_specs) and (cfg.residual_mult != 1.0 or cfg.streams
                                                      or cfg.post_norm):
             raise ValueError("output biases ride on the plain residual add (multiplier 1)")
+        if cfg.sandwich and (cfg.residual_mult != 1.0 or cfg.streams or cfg.post_norm or cfg.loop
+                             or cfg.norm_groups != 1 or any(s.bias or s.shift
+                                                            for s in cfg.layer_specs)):
+            raise ValueError("sandwich norms run on the plain residual, without a loop")
         if cfg.streams and cfg.loop and (cfg.loop_entry or cfg.loop_add):
             raise ValueError("a loop that re-reads the embedding runs on the plain residual")
         for i, spec in enumerate(cfg.layer_specs):
@@ -179,8 +191,27 @@ class HybridLM(TransformerLM):
                 y = prev = None
         return H.hyper_mix(xs, y, prev, self._sum_streams, None)
 
+    def _sandwich_layers(self, x: torch.Tensor, b: DeviceBatch, kv_caches) -> torch.Tensor:
+        """Layers with a norm before and after every sublayer."""
+        cfg = self.cfg
+        eps, off = cfg.norm_eps, cfg.norm_offset
+        step = self._step_view(b, kv_caches.block_size)
+        h = H.resadd_groupnorm(x, None, self.layers[0]["norm1"], 1, eps, w_offset=off)
+        for li, (spec, lp) in enumerate(zip(cfg.layer_specs, self.layers)):
+            following = self.layers[li + 1]["norm1"] if li + 1 < len(self.layers) else None
+            y = MIXERS[spec.kind](spec, lp, h, step, kv_caches.entries[li], eps)
+            h = H.sandwich_add(x, y, lp["norm1b"], eps, lp["norm2"] if spec.ff else following, off)
+            if spec.ff:
+                y = FEED_FORWARDS[spec.ff_kind](spec, lp, h)
+                h = H.sandwich_add(x, y, lp["norm2b"], eps, following, off)
+            if self.layer_trace is not None:
+                self.layer_trace.append(x.clone())
+        return x
+
     def forward_layers(self, x, b: DeviceBatch, kv_caches) -> torch.Tensor:
         cfg, p = self.cfg, self.params
+        if cfg.sandwich:
+            return self._sandwich_layers(x, b, kv_caches)
         if cfg.post_norm:
             return self._postnorm_layers(x, b, kv_caches)
         if cfg.streams:
@@ -275,6 +306,8 @@ class HybridLM(TransformerLM):
                     fused[id(lp["w_up"])] = "bias_gelu"
                 elif spec.ff_kind == "clamp_swish":
                     fused[id(lp["w_gu"])] = "clamp_mul"
+                elif spec.ff_kind == "gated_relu":
+                    fused[id(lp["w_gu"])] = "relu_mul"
                 elif spec.ff_kind == "gated_silu":
                     fused[id(lp["w_gu"])] = "silu_mul"
                 elif spec.shared_ff and spec.expert_act == "gelu_erf":

@@ -19,6 +19,7 @@ import torch
 
 from ..ops import hybrid as H
 from .configs import LayerSpec
+from .weights import input_width
 
 
 @dataclass
@@ -40,7 +41,7 @@ class StepView:
         all layers that rotate alike; None without rotation."""
         if not spec.rot_dims:
             return None
-        key = (spec.rot_dims, spec.rot_base)
+        key = (spec.rot_dims, spec.rot_base, spec.rot_llama3)
         t = self.tables.get(key)
         if t is None:
             t = self.tables[key] = H.rotation_table(self.positions, lp["rot_freq"])
@@ -63,12 +64,27 @@ def derive_constants(spec: LayerSpec, lp: dict, device) -> None:
     elif spec.kind == "lightning":
         lp["decays"] = torch.tensor(spec.decays, dtype=torch.float64).float().to(device)
     elif spec.kind in ("retention", "rope_attention"):
-        lp["rot_freq"] = yarn_frequencies(spec.rot_dims, spec.rot_base)[0].to(device)
+        f = yarn_frequencies(spec.rot_dims, spec.rot_base)[0]
+        if spec.rot_llama3:
+            from ..ops.reference import rope_scaled_inv_freq
+            factor, low, high, orig = spec.rot_llama3
+            f = rope_scaled_inv_freq(f, {"rope_type": "llama3", "factor": factor,
+                                         "low_freq_factor": low, "high_freq_factor": high,
+                                         "original_max_position_embeddings": orig})
+        lp["rot_freq"] = f.to(device)
         if spec.kind == "retention":
             # powers 0 .. RETENTION_CHUNK of every head's decay, each rounded once
             n = torch.arange(H.RETENTION_CHUNK + 1, dtype=torch.float64)
             dec = torch.tensor(spec.decays, dtype=torch.float64)
             lp["decay_pow"] = torch.pow(dec[:, None], n[None, :]).float().contiguous().to(device)
+    elif spec.kind == "ssd":
+        for k in ("conv_w", "conv_b", "dt_bias", "skip"):
+            lp[k] = lp[k].float().contiguous()
+        lp["rate"] = torch.exp(lp["A_log"].double()).float().contiguous()
+    elif spec.kind == "side_by_side":
+        for side, s in (("left", spec.left), ("right", spec.right)):
+            lp[side] = {k[len(side) + 1:]: v for k, v in lp.items() if k.startswith(side + ".")}
+            derive_constants(s, lp[side], device)
     elif spec.kind == "parallel":
         freq, mscale = yarn_frequencies(spec.left.rot_dims, spec.left.rot_base,
                                         spec.left.rot_scaling)
@@ -257,29 +273,78 @@ def retention_mixer(spec: LayerSpec, lp: dict, h, step: StepView, cache, eps: fl
     return H.linear_out(o, lp["wo"])
 
 
-def rope_attention_mixer(spec: LayerSpec, lp: dict, h, step: StepView, cache, eps: float):
-    """Grouped-query softmax attention over a sliding window plus kept first positions, partly
-    rotated q and k, optional biases, values optionally tied to the unrotated keys. The output
-    projection's bias is added with the residual (``HybridLM.forward_layers``)."""
+def rope_attention_heads(spec: LayerSpec, lp: dict, proj, step: StepView, cache, eps: float, dtype):
+    """The concatenated heads [T, H*dv] (storage dtype) of ``rope_attention_mixer``, from the fp32
+    input projection [T, q | k | v | output gate] (v absent with tied values; k and v absent when
+    they are another layer's, whose cache ``cache`` then is; the gate only with ``out_gate``)."""
     kc, vc = cache
-    proj = H.linear_any(h, lp["w_in"])                       # fp32 [T, q | k (| v)]
+    own = spec.kv_from < 0
     q = H.rope_prepare(proj, lp.get("b_in"), step.rotation(spec, lp), spec.rot_dims, spec.heads,
-                       spec.kv_heads, spec.dim, spec.vdim, kc, vc, step.slot_mapping, h.dtype,
-                       spec.tied_values)
+                       spec.kv_heads, spec.dim, spec.vdim, kc, vc, step.slot_mapping, dtype,
+                       spec.tied_values, spec.rot_adjacent, own)
+    gate = None
+    if spec.out_gate:
+        g0 = proj.shape[1] - spec.heads * spec.vdim
+        gate = proj[:, g0:]
     # a window no shorter than the step's longest context masks nothing
     ctx = max(1, step.max_context)
     win = min(spec.window, ctx)
-    o = H.window_attention(q, kc, vc, spec.dim, spec.vdim, spec.heads, spec.kv_heads,
-                           step.cu_seqlens, step.max_seqlen, step.positions, step.block_tables,
-                           step.block_size, win, spec.scale,
-                           keep_first=min(spec.keep_first, ctx) if win < ctx else 0)
-    return H.linear_out(o, lp["wo"])
+    return H.window_attention(q, kc, vc, spec.dim, spec.vdim, spec.heads, spec.kv_heads,
+                              step.cu_seqlens, step.max_seqlen, step.positions,
+                              step.block_tables, step.block_size, win, spec.scale, gate=gate,
+                              keep_first=min(spec.keep_first, ctx) if win < ctx else 0)
+
+
+def ssd_heads(spec: LayerSpec, lp: dict, proj, step: StepView, cache, eps: float, dtype):
+    """The normed read-outs [T, H*dv] (storage dtype) of ``ssd_mixer``, from the fp32 input
+    projection [T, gate z | x | B | C | dt]."""
+    state, conv = cache
+    inner = spec.heads * spec.vdim
+    y = H.ssd(proj[:, inner:], lp["conv_w"], lp["conv_b"], lp["dt_bias"], lp["rate"], lp["skip"],
+              state, conv, step.state_slots, step.cu_seqlens, step.max_seqlen, step.positions,
+              spec.heads, spec.dim, spec.vdim, spec.groups, dtype)
+    return H.gated_rmsnorm(y, proj[:, :inner], lp["o_norm"], eps, spec.norm_parts)
+
+
+def rope_attention_mixer(spec: LayerSpec, lp: dict, h, step: StepView, cache, eps: float):
+    """Grouped-query softmax attention over a sliding window plus kept first positions, partly
+    rotated q and k, optional biases, values optionally tied to the unrotated keys, an optional
+    elementwise output gate, optionally another layer's keys and values. The output projection's
+    bias is added with the residual (``HybridLM.forward_layers``)."""
+    proj = H.linear_any(h, lp["w_in"])                       # fp32 [T, q (| k (| v)) (| gate)]
+    return H.linear_out(rope_attention_heads(spec, lp, proj, step, cache, eps, h.dtype), lp["wo"])
+
+
+def ssd_mixer(spec: LayerSpec, lp: dict, h, step: StepView, cache, eps: float):
+    """State-space recurrence with a decay and a step size per token and head: short causal
+    convolution, recurrence and skip, SiLU gate, RMS norm in parts. Everything between the
+    convolution and the norm runs in fp32."""
+    proj = H.linear_any(h, lp["w_in"])
+    return H.linear_out(ssd_heads(spec, lp, proj, step, cache, eps, h.dtype), lp["wo"])
+
+
+HEADS = {"rope_attention": rope_attention_heads, "ssd": ssd_heads}
+
+
+def side_by_side_mixer(spec: LayerSpec, lp: dict, h, step: StepView, cache, eps: float):
+    """Two mixers on the same input through one fused input projection. Each output projection is
+    RMS-normed with a weight of its own; the result is the mean of the two, formed where it is
+    consumed (``H.SideBySide``)."""
+    l, r = spec.left, spec.right
+    lp_l, lp_r = lp["left"], lp["right"]
+    proj = H.linear_any(h, lp["w_in"])
+    nl = input_width(l)
+    ol = HEADS[l.kind](l, lp_l, proj[:, :nl], step, cache[:2], eps, h.dtype)
+    yl = H.linear_any(ol, lp_l["wo"])
+    outr = HEADS[r.kind](r, lp_r, proj[:, nl:], step, cache[2:], eps, h.dtype)
+    return H.SideBySide(yl, H.linear_out(outr, lp_r["wo"]), lp_l["out_norm"], lp_r["out_norm"], eps)
 
 
 MIXERS = {"attention": attention_mixer, "hgrn2": hgrn2_mixer,
           "latent_attention": latent_attention_mixer, "talk_attention": talk_attention_mixer,
           "gla": gla_mixer, "lightning": lightning_mixer, "parallel": parallel_mixer,
-          "retention": retention_mixer, "rope_attention": rope_attention_mixer}
+          "retention": retention_mixer, "rope_attention": rope_attention_mixer,
+          "ssd": ssd_mixer, "side_by_side": side_by_side_mixer}
 
 
 # ----------------------------------------------------------------------------- feed-forwards
@@ -297,12 +362,13 @@ def prepare_feed_forward(spec: LayerSpec, params: dict, pre: str) -> None:
     from ..ops.reference import interleave_gate_up
     w = params.get(pre + "w_down")
     if (not spec.ff or w is None or pre + "ff_tuned" in params or w.dtype != torch.bfloat16
-            or not w.is_cuda or spec.ff_kind not in ("gelu", "moe", "gated_silu", "clamp_swish")
+            or not w.is_cuda
+            or spec.ff_kind not in ("gelu", "moe", "gated_silu", "clamp_swish", "gated_relu")
             or w.shape[-2] % 64 or spec.ff % 64 or spec.shared_ff % 64):
         return
     if spec.ff_kind == "gelu":
         params[pre + "b_up"] = torch.zeros(spec.ff, dtype=w.dtype, device=w.device)
-    elif spec.ff_kind in ("gated_silu", "clamp_swish"):
+    elif spec.ff_kind in ("gated_silu", "clamp_swish", "gated_relu"):
         if spec.ff_kind == "clamp_swish":            # read by the GEMM's epilogue
             params[pre + "act_limit"] = torch.full((1,), spec.act_limit, dtype=torch.float32,
                                                    device=w.device)
@@ -343,6 +409,15 @@ def gated_silu_ff(spec: LayerSpec, lp: dict, h):
     return H.linear_any(act, lp["w_down"])
 
 
+def gated_relu_ff(spec: LayerSpec, lp: dict, h):
+    if "ff_tuned" in lp:
+        from .. import ops
+        act = ops.linear(h, lp["w_gu"], epi="relu_mul")
+    else:
+        act = H.act_mul(H.linear_any(h, lp["w_gu"]), spec.ff, h.dtype, "relu_mul")
+    return H.linear_out(act, lp["w_down"])
+
+
 def clamp_swish_ff(spec: LayerSpec, lp: dict, h):
     """down(g sigmoid(1.702 g) (u + 1)), g = min(gate, limit), u = clamp(up, -limit, limit)."""
     if "ff_tuned" in lp:
@@ -358,7 +433,14 @@ def moe_ff(spec: LayerSpec, lp: dict, h):
     """Routed gated-SiLU experts + identity experts + a gated shared expert, summed in fp32;
     with ``router`` = ``logit_topk``: biased logits, softmax over the chosen, ungated exact-GELU
     experts and an always-on shared expert; with ``router`` = ``group_score``: group-limited
-    choice, scaled scores, clamped-swish experts."""
+    choice, scaled scores, clamped-swish experts; with ``router`` = ``sigmoid``: a chosen
+    expert's sigmoid score weighs its input, and the sum is formed where it is consumed
+    (``H.RoutedRows``)."""
+    if spec.router == "sigmoid":
+        tw, ti = H.sigmoid_router(h, lp["router"], spec.top)
+        shared = (lp["ws_gu"], lp["ws_down"]) if spec.shared_ff else None
+        return H.moe_weighed_inputs(h, lp["w_gu"], lp["w_down"], tw, ti, shared,
+                                    tuned="ff_tuned" in lp)
     if spec.router == "group_score":
         tw, ti, _ = H.score_router(h, lp["router"], None, spec.top, 0, spec.router_groups,
                                    spec.router_keep, spec.router_scale)
@@ -395,4 +477,5 @@ def moe_ff(spec: LayerSpec, lp: dict, h):
 
 
 FEED_FORWARDS = {"gated_gelu": gated_gelu_ff, "gelu": gelu_ff, "moe": moe_ff,
-                 "gated_silu": gated_silu_ff, "clamp_swish": clamp_swish_ff}
+                 "gated_silu": gated_silu_ff, "clamp_swish": clamp_swish_ff,
+                 "gated_relu": gated_relu_ff}

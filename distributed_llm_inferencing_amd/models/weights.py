@@ -27,6 +27,27 @@ from ..ops.reference import interleave_gate_up
 INIT_STD = 0.02
 
 
+def input_width(s) -> int:
+    """Rows of the fused input projection of a mixer that can stand alone or beside another."""
+    H, d, dv = s.heads, s.dim, s.vdim
+    if s.kind == "ssd":
+        return H * dv + s.conv_channels + H
+    own = s.kv_heads * (d + (0 if s.tied_values else dv)) if s.kv_from < 0 else 0
+    return H * d + own + (H * dv if s.out_gate else 0)
+
+
+def _inner_shapes(s, D: int) -> Dict[str, tuple]:
+    """The other tensors of such a mixer."""
+    out = {"wo": (D, s.heads * s.vdim)}
+    if s.kind == "ssd":
+        out.update({"o_norm": (s.heads * s.vdim,), "conv_w": (s.conv_channels, s.taps),
+                    "conv_b": (s.conv_channels,), "dt_bias": (s.heads,), "A_log": (s.heads,),
+                    "skip": (s.heads,)})
+    elif s.bias:
+        out.update({"b_in": (input_width(s),), "b_out": (D,)})
+    return out
+
+
 def hybrid_layer_shapes(cfg: ModelConfig, i: int) -> Dict[str, tuple]:
     """In-memory tensors of hybrid layer ``i`` (``layers.{i}.``), projections that read the
     same input fused row-wise:
@@ -68,7 +89,17 @@ def hybrid_layer_shapes(cfg: ModelConfig, i: int) -> Dict[str, tuple]:
       rope_attention:   w_in [(H + G)*d (+ G*dv), D] = q | k (| v, absent with ``tied_values``),
                         wo [D, H*dv]; with ``bias``: b_in, b_out [D]
         clamp_swish:    w_gu [2F, D] = gate | up, w_down [D, F]
-    Post-norm designs add the norms' biases norm1_b / norm2_b [D]; with a per-layer token input
+      rope_attention with ``kv_from``: w_in holds the q part only; with ``out_gate``: H*dv gate
+                        rows follow
+      ssd:              w_in [2*H*dv + 2*G*d + H, D] = gate z | x | B | C | dt, wo [D, H*dv],
+                        o_norm [H*dv], fp32: conv_w [channels, taps], conv_b [channels] (channels
+                        = x | B | C), dt_bias [H], A_log [H], skip [H]
+      side_by_side:     w_in = the left mixer's | the right mixer's; their other tensors under
+                        ``left.`` / ``right.``, with out_norm [D] each
+        gated_relu:     w_gu [2F, D] = gate | up, w_down [D, F]
+        moe, router ``sigmoid``: router [E, D], w_gu [E, 2F, D], w_down [E, D, F], shared
+                        ws_gu [2Fs, D], ws_down [D, Fs]
+    Sandwich-norm designs add norm1b / norm2b [D] (behind the sublayers). Post-norm designs add the norms' biases norm1_b / norm2_b [D]; with a per-layer token input
     of width s: side_gate [s, D], side_proj [D, s], side_norm [D]. With hyper-connections over
     S streams every sublayer has hc1 / hc2 fp32 [S + S + S*S] = read weights | write weights |
     stream mix [from, to]."""
@@ -114,11 +145,14 @@ def hybrid_layer_shapes(cfg: ModelConfig, i: int) -> Dict[str, tuple]:
                     p + "wo": (D, l.heads * l.vdim + r.heads * r.vdim)})
     elif s.kind == "retention":
         out.update({p + "w_in": (2 * H * (d + dv), D), p + "wo": (D, H * dv)})
-    elif s.kind == "rope_attention":
-        n_in = (H + s.kv_heads) * d + (0 if s.tied_values else s.kv_heads * dv)
-        out.update({p + "w_in": (n_in, D), p + "wo": (D, H * dv)})
-        if s.bias:
-            out.update({p + "b_in": (n_in,), p + "b_out": (D,)})
+    elif s.kind in ("rope_attention", "ssd"):
+        out[p + "w_in"] = (input_width(s), D)
+        out.update({p + k: v for k, v in _inner_shapes(s, D).items()})
+    elif s.kind == "side_by_side":
+        out[p + "w_in"] = (input_width(s.left) + input_width(s.right), D)
+        for side, m in (("left.", s.left), ("right.", s.right)):
+            out.update({p + side + k: v for k, v in _inner_shapes(m, D).items()})
+            out[p + side + "out_norm"] = (D,)
     else:
         raise ValueError(f"unknown mixer kind '{s.kind}'")
     if cfg.streams:
@@ -126,6 +160,10 @@ def hybrid_layer_shapes(cfg: ModelConfig, i: int) -> Dict[str, tuple]:
         out[p + "hc1"] = (n,)
         if s.ff:
             out[p + "hc2"] = (n,)
+    if cfg.sandwich:
+        out[p + "norm1b"] = (D,)
+        if s.ff:
+            out[p + "norm2b"] = (D,)
     if cfg.post_norm:
         out[p + "norm1_b"] = (D,)
         if s.ff:
@@ -138,13 +176,15 @@ def hybrid_layer_shapes(cfg: ModelConfig, i: int) -> Dict[str, tuple]:
                     p + "w_up": (s.experts, s.ff, D), p + "w_down": (s.experts, D, s.ff)})
         if s.shared_ff:
             out.update({p + "ws_up": (s.shared_ff, D), p + "ws_down": (D, s.shared_ff)})
-    elif s.ff and s.ff_kind in ("gated_gelu", "gated_silu", "clamp_swish"):
+    elif s.ff and s.ff_kind in ("gated_gelu", "gated_silu", "clamp_swish", "gated_relu"):
         out.update({p + "norm2": (D,), p + "w_gu": (2 * s.ff, D), p + "w_down": (D, s.ff)})
     elif s.ff and s.ff_kind == "gelu":
         out.update({p + "norm2": (D,), p + "w_up": (s.ff, D), p + "w_down": (D, s.ff)})
-    elif s.ff and s.ff_kind == "moe" and s.router == "group_score":
+    elif s.ff and s.ff_kind == "moe" and s.router in ("group_score", "sigmoid"):
         out.update({p + "norm2": (D,), p + "router": (s.experts, D),
                     p + "w_gu": (s.experts, 2 * s.ff, D), p + "w_down": (s.experts, D, s.ff)})
+        if s.shared_ff:
+            out.update({p + "ws_gu": (2 * s.shared_ff, D), p + "ws_down": (D, s.shared_ff)})
     elif s.ff and s.ff_kind == "moe":
         n = s.experts + s.identity
         out.update({p + "norm2": (D,), p + "router": (n + (1 if s.shared_ff else 0), D),
@@ -223,7 +263,8 @@ def stage_param_shapes(cfg: ModelConfig, layer_start: int, layer_end: int, first
 
 def _is_norm_weight(name: str) -> bool:
     return name.endswith(("attn_norm", "mlp_norm", "final_norm", "ln1_w", "ln2_w", "norm1",
-                          "norm2", "q_norm", "k_norm", "c_norm", "o_norm", "side_norm"))
+                          "norm2", "q_norm", "k_norm", "c_norm", "o_norm", "side_norm",
+                          "norm1b", "norm2b", "out_norm"))
 
 
 def _is_bias(name: str) -> bool:
@@ -244,7 +285,8 @@ def random_init(shapes: Dict[str, tuple], device, dtype=torch.bfloat16, seed: in
             out[name] = _hybrid_init(name, shape, dev, dtype, seed)
         elif _is_norm_weight(name):
             # a design that stores its layer norms' weights as offsets starts them at zero
-            v = norm_value if name.endswith(("norm1", "norm2", "final_norm")) else 1.0
+            v = norm_value if name.endswith(("norm1", "norm2", "norm1b", "norm2b",
+                                             "final_norm")) else 1.0
             out[name] = torch.full(shape, v, dtype=dtype, device=dev)
         elif _is_bias(name):
             out[name] = torch.zeros(shape, dtype=dtype, device=dev)
@@ -286,6 +328,17 @@ def _hybrid_init(name: str, shape: tuple, dev, dtype, seed: int) -> torch.Tensor
         t = torch.cat([-1.0 + 0.5 * torch.randn(H, generator=g),
                        3.0 + 1.0 * torch.randn(H, generator=g)])
         return t.to(dev, torch.float32)
+    if name.endswith(".A_log"):                  # ssd: decay rates between 1 and 16
+        return torch.log(1.0 + 15.0 * torch.rand(shape, generator=g)).to(dev, torch.float32)
+    if name.endswith(".dt_bias"):                # ... step sizes between 0.001 and 0.1
+        dt = torch.exp(torch.rand(shape, generator=g) * 4.605 - 6.908)
+        return (dt + torch.log(-torch.expm1(-dt))).to(dev, torch.float32)
+    if name.endswith(".skip"):
+        return torch.ones(shape).to(dev, torch.float32)
+    if name.endswith(".conv_w"):
+        return (torch.randn(shape, generator=g) / shape[-1] ** 0.5).to(dev, torch.float32)
+    if name.endswith(".conv_b"):
+        return (0.02 * torch.randn(shape, generator=g)).to(dev, torch.float32)
     if name.endswith(".a_b"):
         # decays sigmoid(z)^(1/tau) spread between fast and slow channels
         return (1.0 + 2.0 * torch.randn(shape, generator=g)).to(dev, dtype)
@@ -643,4 +696,50 @@ def from_bamudra_state_dict(cfg: ModelConfig, sd, dtype=torch.bfloat16) -> Dict[
             out[p + "norm2"] = cv(sd[a + "norm2"])
             out[p + "w_gu"] = cv(torch.cat([sd[f + "gate"], sd[f + "up"]], 0))
             out[p + "w_down"] = cv(sd[f + "down"])
+    return _checked(cfg, out)
+
+
+# ----------------------------------------------------------------------------- Lutovik files
+def from_lutovik_state_dict(cfg: ModelConfig, sd, dtype=torch.bfloat16) -> Dict[str, torch.Tensor]:
+    """Convert a Lutovik checkpoint (tensor names ``embed``, ``head``, ``final.norm``,
+    ``l<i>.norm1|norm1b|norm2|norm2b``, ``l<i>.mix.q|k|v|o`` of an attention layer,
+    ``l<i>.mix.left.q|k|v|g|o|out`` and ``l<i>.mix.right.in|conv|conv.b|dt_bias|A_log|D|norm|o|out``
+    of a parallel one, ``l<i>.mlp.gate|up|down`` or ``l<i>.mlp.router|e<j>.*|shared.*``; linear
+    weights [out, in]) into the layout of ``hybrid_layer_shapes``: projections that read the same
+    input are stacked, the experts are stacked, what enters the recurrence besides projections
+    is kept in fp32. Norm weights stay as stored (offsets from one)."""
+    cv = lambda t: t.detach().to(dtype).contiguous()  # noqa: E731
+    f32 = lambda t: t.detach().float().contiguous()  # noqa: E731
+    out = {"embed": cv(sd["embed"]), "lm_head": cv(sd["head"]), "final_norm": cv(sd["final.norm"])}
+    for i, s in enumerate(cfg.layer_specs):
+        a, p = f"l{i}.", f"layers.{i}."
+        m, f = a + "mix.", a + "mlp."
+        out[p + "norm1"], out[p + "norm1b"] = cv(sd[a + "norm1"]), cv(sd[a + "norm1b"])
+        if s.kind == "side_by_side":
+            lt, rt = m + "left.", m + "right."
+            out[p + "w_in"] = cv(torch.cat([sd[lt + n] for n in "qkvg"] + [sd[rt + "in"]], 0))
+            for side, t in (("left.", lt), ("right.", rt)):
+                out[p + side + "wo"], out[p + side + "out_norm"] = cv(sd[t + "o"]), cv(sd[t + "out"])
+            q = p + "right."
+            out[q + "o_norm"] = cv(sd[rt + "norm"])
+            for name, src in (("conv_w", "conv"), ("conv_b", "conv.b"), ("dt_bias", "dt_bias"),
+                              ("A_log", "A_log"), ("skip", "D")):
+                out[q + name] = f32(sd[rt + src])
+        else:
+            out[p + "w_in"] = cv(torch.cat([sd[m + n] for n in ("q" if s.kv_from >= 0 else "qkv")], 0))
+            out[p + "wo"] = cv(sd[m + "o"])
+        if not s.ff:
+            continue
+        out[p + "norm2"], out[p + "norm2b"] = cv(sd[a + "norm2"]), cv(sd[a + "norm2b"])
+        if s.ff_kind == "gated_relu":
+            out[p + "w_gu"] = cv(torch.cat([sd[f + "gate"], sd[f + "up"]], 0))
+            out[p + "w_down"] = cv(sd[f + "down"])
+            continue
+        out[p + "router"] = cv(sd[f + "router"])
+        out[p + "w_gu"] = cv(torch.stack([torch.cat([sd[f"{f}e{e}.gate"], sd[f"{f}e{e}.up"]], 0)
+                                          for e in range(s.experts)]))
+        out[p + "w_down"] = cv(torch.stack([sd[f"{f}e{e}.down"] for e in range(s.experts)]))
+        if s.shared_ff:
+            out[p + "ws_gu"] = cv(torch.cat([sd[f + "shared.gate"], sd[f + "shared.up"]], 0))
+            out[p + "ws_down"] = cv(sd[f + "shared.down"])
     return _checked(cfg, out)

@@ -238,8 +238,8 @@ def _gemm_native(x, w, epi: str, bias=None, out=None, plan: Optional[G.GemmPlan]
 
 def linear(x, w, bias=None, epi: str = "none", out=None):
     """y = epi(x @ w.T (+bias)). epi in {none, f32, silu_mul, bias_gelu, bias, gelu_erf,
-    clamp_mul}. silu_mul and clamp_mul expect the 16-row interleaved gate/up weight and return
-    width N/2; clamp_mul takes its limit as ``bias``, one fp32 number on the device."""
+    clamp_mul, relu_mul}. silu_mul, clamp_mul and relu_mul expect the 16-row interleaved gate/up
+    weight and return width N/2; clamp_mul takes its limit as ``bias``, one fp32 number on the device."""
     if bias is not None and epi == "none":
         epi = "bias"
     if isinstance(x, NormedRows):
@@ -261,6 +261,9 @@ def linear(x, w, bias=None, epi: str = "none", out=None):
         elif epi == "clamp_mul":
             gu = torch.cat(R.split_gate_up(R.linear(x, w, out_dtype=torch.float32)), -1)
             y = R.clamp_swish_mul(gu, w.shape[-2] // 2, float(bias), x.dtype)
+        elif epi == "relu_mul":
+            g, u = R.split_gate_up(R.linear(x, w, out_dtype=torch.float32))
+            y = (torch.relu(g) * u).to(x.dtype)
         elif epi == "gelu_erf":
             y = torch.nn.functional.gelu(R.linear(x, w, out_dtype=torch.float32)).to(x.dtype)
         else:
@@ -792,6 +795,34 @@ def moe_mlp(x, w_gu, w_down, topk_w, topk_ids, expert_offset: int = 0,
     out = torch.empty_like(x)
     _native_call("dli_moe_combine", _p(out), _p(y), _p(topk_w), _p(pos), T, k, D, _st())
     return out
+
+
+def moe_rows(x, w_gu, w_down, topk_w, topk_ids):
+    """Experts whose weight multiplies their input, not their output: (y bf16 [T * k, D], pos int32
+    [T * k]) with y[pos[t * k + j]] = expert_j(topk_w[t, j] * x[t]) for gated-SiLU experts in the
+    interleaved layout; the consumer sums a token's rows. GPU only."""
+    from .hybrid import weighed_rows
+    T, D = x.shape
+    E, F2, _ = w_gu.shape
+    n = T * topk_ids.shape[1]
+    offsets, pos, xp = weighed_rows(x, topk_w, topk_ids, E)
+    act = torch.empty(max(n, 1), F2 // 2, dtype=x.dtype, device=x.device)
+    y = torch.empty(max(n, 1), D, dtype=x.dtype, device=x.device)
+    p_gu = p_dn = None
+    rows = n
+    if n >= _MOE_PREFILL_ROWS * E and not torch.cuda.is_current_stream_capturing():
+        # prefill-sized expert GEMMs: as in ``moe_mlp``
+        offs = offsets.tolist()
+        rows = max(b - a for a, b in zip(offs[:-1], offs[1:]))
+        p_gu = p_dn = G.GemmPlan("dli", G.MOE_PREFILL_TILE, 1)
+    p_gu = p_gu or G.grouped_plan(n, F2, D, "silu_mul", E)
+    p_dn = p_dn or G.grouped_plan(n, D, F2 // 2, "none", E)
+    if rows > 0:
+        _gemm_native(xp, w_gu, "silu_mul", out=act, groups=E, group_off=offsets,
+                     rows_per_group=rows, plan=p_gu)
+        _gemm_native(act, w_down, "none", out=y, groups=E, group_off=offsets, rows_per_group=rows,
+                     plan=p_dn)
+    return y, pos
 
 
 def moe_slab_plan(p: Optional[G.GemmPlan]) -> bool:

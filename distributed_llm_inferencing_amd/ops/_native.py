@@ -109,8 +109,16 @@ _SIGS = {
     # rotated designs (rotary.hip, retention.hip, swa_attention.hip)
     "dli_swa_attention": [P, I, P, L, P, L, P, I, P, P, P, I, I, I, I, I, I, I, I, I, F, P, P],
     "dli_swa_attention_workspace_bytes": [I, I, I, I, I, I, I],
+    "dli_sandwich_add": [P, P, I, I, L, P, I, P, P, F, P, I, I, P, P, P, I, I, F, F, I, P],
+    "dli_gated_rmsnorm": [P, P, I, P, I, P, I, I, I, F, I, P],
+    "dli_sigmoid_router": [P, P, P, I, P, I, I, I, I, I, P],
+    "dli_moe_scatter_weighed": [P, P, I, P, P, I, I, I, I, P],
+    "dli_ssd_conv": [P, I, P, P, I, P, P, P, P, P, I, I, I, I, P],
+    "dli_ssd_chunks": [P, I, P, I, P, P, P, P, P, P, P, P, I, I, I, I, I, I, P],
+    "dli_ssd_walk": [P, I, P, I, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, P],
+    "dli_ssd_step": [P, I, P, P, I, P, P, P, P, P, P, P, P, P, I, I, I, I, I, P],
     "dli_rotation_table": [P, P, P, I, I, P],
-    "dli_rope_prepare": [P, I, P, P, I, I, I, I, I, I, I, P, P, P, P, I, P],
+    "dli_rope_prepare": [P, I, P, P, I, I, I, I, I, I, I, I, P, P, P, P, I, P],
     "dli_retention": [P, I, P, I, P, I, F, F, P, P, P, P, P, I, I, I, I, I, I, I, P, I, I, P],
 }
 

@@ -88,12 +88,12 @@ def tile_ok(tile: int, epi: str) -> bool:
     which must therefore be a multiple of 32."""
     if epi == "res":
         return tile in GEMV_RES_TILES
-    if epi in ("gelu_erf", "clamp_mul") and tile in (34, 41, 45, 55):
+    if epi in ("gelu_erf", "clamp_mul", "relu_mul") and tile in (34, 41, 45, 55):
         return False            # the 4-wave families are built without these epilogues
     if tile in (29, 58, 59):
         return epi == "silu_mul"
     if tile in GEMV_TILES:
-        return epi != "clamp_mul" and (epi != "silu_mul" or tile in (31, 33))
+        return epi not in ("clamp_mul", "relu_mul") and (epi != "silu_mul" or tile in (31, 33))
     if epi not in PAIR_EPIS:
         return True
     if tile == 26:              # the straddling gate/up pair meets through LDS
@@ -105,9 +105,9 @@ def tile_ok(tile: int, epi: str) -> bool:
 # "splitk": a plain GEMM whose fp32 partial slabs feed a fused reduce (ops.linear_add_rmsnorm,
 # ops.linear_rope_cache); planned/tuned separately (a non-split winner runs unfused).
 EPI = {"none": 0, "f32": 1, "silu_mul": 2, "bias_gelu": 3, "bias": 4, "splitk": 0,
-       "slab16": 5, "gelu_erf": 6, "clamp_mul": 7}
+       "slab16": 5, "gelu_erf": 6, "clamp_mul": 7, "relu_mul": 8}
 # epilogues over the interleaved gate/up weight: the output is half as wide
-PAIR_EPIS = ("silu_mul", "clamp_mul")
+PAIR_EPIS = ("silu_mul", "clamp_mul", "relu_mul")
 # tiles whose slab-only split-K call can store fp16 partials (EPI "slab16": the generic tile
 # family and the 8-phase kernels); the fused consumers then read half the bytes. The
 # weight-streaming GEMVs and the 4-wave family keep fp32 slabs.
@@ -176,7 +176,7 @@ def _heuristic(M: int, N: int, K: int, epi: str) -> GemmPlan:
         # residual-adding GEMV (full K): 4 rows a workgroup, 8 K-steps in flight per lane
         # (1024 workgroups on a 4096-wide projection)
         return GemmPlan("dli", 56, 1)
-    if M <= GEMV_MAX_M and epi != "clamp_mul":      # (the GEMVs are built without it)
+    if M <= GEMV_MAX_M and epi not in ("clamp_mul", "relu_mul"):    # (the GEMVs have neither)
         # batch-1 / tiny batches: stream the weights (gemv_kernel) with enough workgroups
         # (>= 512, two per CU) to keep ~64 KB of loads in flight per CU
         # gate/up at M <= 2: the 16-row SiLU grid (tile 29) 39.5 / 43.3 vs 49.0 / 51.0 us for

@@ -11,6 +11,7 @@ exact mode) is the dtype of the weights; kernels take it as ``dt``.
 from __future__ import annotations
 
 import os
+from dataclasses import dataclass
 from typing import Optional
 
 import torch
@@ -20,6 +21,7 @@ from . import gemm as _gemm
 from . import reference as R
 
 _call = N.call
+_require_native = N.require_native
 _p = N.ptr
 _NOT_SUPPORTED = 801            # hipErrorNotSupported: a launcher declining a shape
 # longest chunk of the retention kernels (the table of decay powers covers it)
@@ -87,8 +89,42 @@ def linear_out(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
     return linear_any(x, w)
 
 
-def rows_of(y: Optional[torch.Tensor]) -> Optional[torch.Tensor]:
-    """[M, N] from what ``linear_out`` returned."""
+@dataclass
+class SideBySide:
+    """Half the sum of two fp32 outputs [T, D], each RMS-normed and times a weight [D] of its own:
+    formed by its consumer (``sandwich_add``, or ``rows_of``). ``right`` may be a GEMM's partial
+    sums (``linear_out``)."""
+    left: torch.Tensor
+    right: torch.Tensor
+    w_left: torch.Tensor
+    w_right: torch.Tensor
+    eps: float
+
+
+@dataclass
+class RoutedRows:
+    """The plain sum of every token's experts' outputs, formed by its consumer
+    (``sandwich_add``, or ``rows_of``): rows ``pos[t * k + j]`` of ``y`` (fp32 or bf16), plus
+    ``shared`` fp32 [T, D] when given."""
+    y: torch.Tensor
+    pos: torch.Tensor
+    k: int
+    shared: Optional[torch.Tensor]
+    tokens: int
+
+
+def rows_of(y) -> Optional[torch.Tensor]:
+    """fp32 [M, N] from what ``linear_out`` or a sublayer returned."""
+    if isinstance(y, SideBySide):
+        if not y.left.is_cuda:
+            return R.mean_of_normed(y.left, rows_of(y.right), y.w_left, y.w_right, y.eps)
+        x = torch.zeros_like(y.left)
+        sandwich_add(x, y, None, 0.0)
+        return x
+    if isinstance(y, RoutedRows):
+        x = torch.zeros(y.tokens, y.y.shape[1], dtype=torch.float32, device=y.y.device)
+        sandwich_add(x, y, None, 0.0)
+        return x
     if y is None or y.dim() == 2:
         return y
     x = torch.empty(y.shape[1:], dtype=torch.float32, device=y.device)
@@ -144,6 +180,8 @@ def resadd_groupnorm(x: torch.Tensor, y: Optional[torch.Tensor], w: Optional[tor
     the grouped RMS norm of the new x times ``w`` times ``gain`` in the storage dtype (None when
     w is None), or unrounded in fp32 with ``out_f32`` (what a token shift reads). ``w_offset``
     is added to the weight in fp32 (weights stored as offsets from one)."""
+    if not isinstance(y, (torch.Tensor, type(None))):
+        y = rows_of(y)
     dtype = dtype or (w.dtype if w is not None else
                       bias.dtype if bias is not None else torch.bfloat16)
     if not x.is_cuda:
@@ -213,13 +251,13 @@ def concat_cast(a: torch.Tensor, b: torch.Tensor, dtype) -> torch.Tensor:
 
 
 _ACT_KINDS = {"gelu_mul": 0, "silu_mul": 1, "gelu": 2, "gelu_erf": 3, "copy": 4,
-              "clamp_swish": 5}
+              "clamp_swish": 5, "relu_mul": 6}
 
 
 def act_mul(gu: torch.Tensor, F_: int, dtype, kind: str = "gelu_mul",
             rows: Optional[torch.Tensor] = None, limit: float = 0.0) -> torch.Tensor:
-    """The feed-forward's middle for an fp32 projection: ``gelu_mul`` / ``silu_mul`` =
-    act(gu[:, :F]) * gu[:, F:2F]; ``gelu`` = gelu_tanh(gu[:, :F]); ``gelu_erf`` = the exact GELU
+    """The feed-forward's middle for an fp32 projection: ``gelu_mul`` / ``silu_mul`` /
+    ``relu_mul`` = act(gu[:, :F]) * gu[:, F:2F]; ``gelu`` = gelu_tanh(gu[:, :F]); ``gelu_erf`` = the exact GELU
     of gu[:, :F]; ``copy`` = gu[:, :F] rounded to the storage dtype; ``clamp_swish`` = g
     sigmoid(1.702 g) (u + 1) with g = min(gu[:, :F], limit), u = clamp(gu[:, F:2F], +-limit).
     ``gu`` may also be a bf16 projection (a tuned GEMM's output) when ``dtype`` is bf16.
@@ -759,17 +797,21 @@ def rotation_table(positions, freq) -> torch.Tensor:
 
 
 def rope_prepare(proj, bias, table, rot_dims: int, H, G, d, dv, kcache, vcache, slots, dtype,
-                 tied: bool):
+                 tied: bool, adjacent: bool = False, own_kv: bool = True):
     """Query / cache preparation of an attention with rotated q and k
     (``reference.rope_prepare``): bias, rotation by the step's table, k and v (or, tied, the
-    unrotated k) to the cache rows; the queries [T, H*d] come back in the storage dtype."""
+    unrotated k) to the cache rows; the queries [T, H*d] come back in the storage dtype.
+    ``adjacent``: rotated pairs are (2i, 2i+1) instead of (i, i + rot_dims/2). Without ``own_kv``
+    the projection holds queries only and nothing is written."""
     if not proj.is_cuda:
         return R.rope_prepare(proj, bias, table, rot_dims, H, G, d, dv, kcache, vcache, slots,
-                              dtype, tied)
+                              dtype, tied, adjacent, own_kv)
     T = proj.shape[0]
     q = torch.empty(T, H * d, dtype=dtype, device=proj.device)
     _call("dli_rope_prepare", _p(proj), proj.stride(0), _p(bias), _p(table), int(rot_dims), T, H,
-          G, d, dv, int(tied), _p(q), _p(kcache), _p(vcache), _p(slots), _dt(dtype), _st())
+          G if own_kv else 0, d, dv, int(tied), int(adjacent), _p(q),
+          _p(kcache) if own_kv else None, _p(vcache) if own_kv else None, _p(slots), _dt(dtype),
+          _st())
     return q
 
 
@@ -805,3 +847,146 @@ def retention(proj, table, rot_dims: int, decay_pow, eps: float, state, slots, c
         rmsnorm_cols(raw, None, eps, gate=proj[:, g0:g0 + H * dv], groups=H, out=out,
                      silu_gate=True)
     return out
+
+
+# ----------------------------------------------------------------------------- sandwich-norm designs
+def sandwich_add(x, y, w_post, eps: float, w_next=None, w_offset: float = 0.0):
+    """In place on the fp32 stream: x += rms(y) * (w_post + w_offset) (x += y without w_post);
+    returns the RMS norm of the new x times (w_next + w_offset) in the storage dtype (None without
+    w_next). y: a sublayer's fp32 output, a GEMM's partial sums (``linear_out``), a
+    ``SideBySide`` or a ``RoutedRows``; one launch for each."""
+    if not x.is_cuda:
+        y = rows_of(y)
+        if w_post is None:
+            x.add_(y)
+            return None
+        return R.sandwich_add(x, y, w_post, eps, w_next, w_offset, w_post.dtype)
+    T, D = x.shape
+    dtype = w_post.dtype if w_post is not None else torch.bfloat16
+    h = torch.empty(T, D, dtype=w_next.dtype, device=x.device) if w_next is not None else None
+    y2 = wl = wr = pos = None
+    k = y_bf16 = 0
+    inner_eps = 0.0
+    if isinstance(y, SideBySide):
+        y, y2, wl, wr, inner_eps = y.right, y.left, y.w_right, y.w_left, y.eps
+        dtype = wl.dtype
+    elif isinstance(y, RoutedRows):
+        y, y2, pos, k = y.y, y.shared, y.pos, y.k
+        y_bf16 = int(y.dtype == torch.bfloat16)
+    slabs = y.dim() == 3
+    if (y2 is not None and y2.shape != x.shape) or y.shape[-1] != D or (
+            pos is None and y.shape[-2] != T):
+        raise ValueError("sandwich_add: the output does not have the stream's shape")
+    _call("dli_sandwich_add", _p(x), _p(y), y.stride(-2), y.shape[0] if slabs else 1,
+          y.stride(0) if slabs else 0, _p(y2), y2.stride(0) if y2 is not None else 0, _p(wl), _p(wr),
+          float(inner_eps), _p(pos), int(k), y_bf16, _p(w_post), _p(w_next), _p(h), T, D,
+          float(eps), float(w_offset), _dt(dtype), _st())
+    return h
+
+
+def gated_rmsnorm(src, gate, w, eps: float, groups: int = 1) -> torch.Tensor:
+    """RMS norm, in ``groups`` equal parts of a row, of src * silu(gate) (fp32 [T, n] both, gate a
+    column slice of a projection), times w [n]; storage dtype of w."""
+    if not src.is_cuda:
+        return R.gated_rmsnorm(src, gate, w, eps, groups, w.dtype)
+    T, n = src.shape
+    out = torch.empty(T, n, dtype=w.dtype, device=src.device)
+    _call("dli_gated_rmsnorm", _p(out), _p(src), src.stride(0), _p(gate), gate.stride(0), _p(w), T,
+          n // groups, int(groups), float(eps), _dt(w.dtype), _st())
+    return out
+
+
+def sigmoid_router(h, w_router, top: int):
+    """(sigmoid scores fp32 [T, top], ids int32 [T, top]) of the ``top`` largest fp32 logits."""
+    if not h.is_cuda:
+        return R.sigmoid_router(h, w_router, top)
+    T, D = h.shape
+    n = w_router.shape[0]
+    w = torch.empty(T, top, dtype=torch.float32, device=h.device)
+    ids = torch.empty(T, top, dtype=torch.int32, device=h.device)
+    _call("dli_sigmoid_router", _p(w), _p(ids), _p(h), h.stride(0), _p(w_router), T, D, n, top,
+          _dt(h.dtype), _st())
+    return w, ids
+
+
+def moe_weighed_inputs(x, w_gu, w_down, topk_w, topk_ids, shared=None, tuned: bool = False):
+    """Experts whose weight multiplies their input: the sum over a token's chosen gated-SiLU
+    experts of expert(weight * row), plus the always-on expert ``shared`` = (ws_gu, ws_down) of
+    the plain row. ``tuned``: bf16 weights in the interleaved gate / up layout of the tuned GEMMs.
+    Returns ``RoutedRows`` (fp32 rows on the CPU). No host synchronisation but for large
+    prefills on the tuned path."""
+    if not x.is_cuda:
+        return R.moe_weighed_inputs_f32(x, w_gu, w_down, topk_w, topk_ids, shared)
+    T, D = x.shape
+    k = topk_ids.shape[1]
+    ys = None
+    if tuned:
+        from . import linear, moe_rows
+        if shared is not None:
+            ys = linear_any(linear(x, shared[0], epi="silu_mul"), shared[1])
+        y, pos = moe_rows(x, w_gu, w_down, topk_w, topk_ids)
+        return RoutedRows(y, pos, k, ys, T)
+    E, F2, _ = w_gu.shape
+    n = T * k
+    if shared is not None:
+        a = act_mul(linear_any(x, shared[0]), shared[0].shape[0] // 2, x.dtype, "silu_mul")
+        ys = linear_any(a, shared[1])
+    offsets, pos, xs = weighed_rows(x, topk_w, topk_ids, E)
+    gu = grouped_linear_any(xs, w_gu, offsets, None, n)
+    act = act_mul(gu, F2 // 2, x.dtype, "silu_mul", rows=offsets[E:])
+    return RoutedRows(grouped_linear_any(act, w_down, offsets, None, n), pos, k, ys, T)
+
+
+def weighed_rows(x, topk_w, topk_ids, E: int):
+    """Rows sorted by expert, each times its weight: (offsets int32 [E + 1], pos int32 [T * k],
+    rows [T * k, D] in the storage dtype with row pos[t * k + j] = topk_w[t, j] * x[t])."""
+    T, D = x.shape
+    k = topk_ids.shape[1]
+    n = T * k
+    offsets = torch.empty(E + 1, dtype=torch.int32, device=x.device)
+    pos = torch.empty(n, dtype=torch.int32, device=x.device)
+    src = torch.empty(max(n, 1), dtype=torch.int32, device=x.device)
+    _call("dli_moe_align", _p(offsets), _p(pos), _p(src), _p(topk_ids), n, k, 0, E, _st())
+    xs = torch.empty(max(n, 1), D, dtype=x.dtype, device=x.device)
+    _call("dli_moe_scatter_weighed", _p(xs), _p(x), x.stride(0), _p(topk_w), _p(pos), n, k, D,
+          _dt(x.dtype), _st())
+    return offsets, pos, xs
+
+
+def ssd(xbcdt, conv_w, conv_b, dt_bias, rate, skip, state, conv, slots, cu_seqlens, max_seqlen,
+        positions, H, N, P, G, dtype) -> torch.Tensor:
+    """State-space recurrence over per-sequence slots (``reference.ssd``): xbcdt fp32
+    [T, x | B | C | dt] (a column slice of a projection); returns y fp32 [T, H*P]."""
+    ch = H * P + 2 * G * N
+    if not xbcdt.is_cuda:
+        return R.ssd(xbcdt[:, :ch], xbcdt[:, ch:ch + H], conv_w, conv_b, dt_bias, rate, skip, state,
+                     conv, slots, cu_seqlens, positions, H, N, P, G)
+    T = xbcdt.shape[0]
+    S = cu_seqlens.shape[0] - 1
+    taps = conv_w.shape[1]
+    y = torch.empty(T, H * P, dtype=torch.float32, device=xbcdt.device)
+    lib = _require_native()
+    if int(max_seqlen) == 1:                 # decode rows: one launch
+        rc = lib.dli_ssd_step(_p(xbcdt), xbcdt.stride(0), _p(conv_w), _p(conv_b), taps, _p(dt_bias),
+                              _p(rate), _p(skip), _p(state), _p(conv), _p(slots), _p(cu_seqlens),
+                              _p(positions), _p(y), S, H, N, P, G, _st())
+        if rc == 0:
+            return y
+        if rc != _NOT_SUPPORTED:
+            raise RuntimeError(f"dli_ssd_step failed with hipError {rc}")
+    chunked = N % 16 == 0 and N <= 256 and P % 4 == 0
+    # the convolved rows: bf16 when serving on the chunk form, else fp32
+    xdt = dtype if chunked else torch.float32
+    xc = torch.empty(T, ch, dtype=xdt, device=xbcdt.device)
+    _call("dli_ssd_conv", _p(xbcdt), xbcdt.stride(0), _p(conv_w), _p(conv_b), taps, _p(conv),
+          _p(slots), _p(cu_seqlens), _p(positions), _p(xc), S, int(max_seqlen), ch, _dt(xdt), _st())
+    dt = xbcdt[:, ch:]
+    if chunked:
+        _call("dli_ssd_chunks", _p(xc), ch, _p(dt), dt.stride(0), _p(dt_bias), _p(rate), _p(skip),
+              _p(state), _p(slots), _p(cu_seqlens), _p(positions), _p(y), S, H, N, P, G, _dt(xdt),
+              _st())
+    else:
+        _call("dli_ssd_walk", _p(xc), ch, _p(dt), dt.stride(0), _p(dt_bias), _p(rate), _p(skip),
+              _p(state), _p(slots), _p(cu_seqlens), _p(positions), _p(y), S, int(max_seqlen), H, N,
+              P, G, _column_block(S, H, N, P, max_seqlen), _st())
+    return y

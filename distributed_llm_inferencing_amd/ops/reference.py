@@ -396,8 +396,8 @@ def group_rmsnorm(x: torch.Tensor, w: torch.Tensor, groups: int, eps: float,
 
 def act_mul(gu: torch.Tensor, F_: int, out_dtype: torch.dtype, kind: str,
             limit: float = 0.0) -> torch.Tensor:
-    """The feed-forward's middle, fp32 in: ``gelu_mul`` / ``silu_mul`` = act(gu[:, :F]) *
-    gu[:, F:2F]; ``gelu`` = gelu_tanh(gu[:, :F]); ``gelu_erf`` = the exact GELU of gu[:, :F];
+    """The feed-forward's middle, fp32 in: ``gelu_mul`` / ``silu_mul`` / ``relu_mul`` =
+    act(gu[:, :F]) * gu[:, F:2F]; ``gelu`` = gelu_tanh(gu[:, :F]); ``gelu_erf`` = the exact GELU of gu[:, :F];
     ``copy`` = gu[:, :F] itself."""
     if kind == "clamp_swish":
         return clamp_swish_mul(gu, F_, limit, out_dtype)
@@ -409,7 +409,8 @@ def act_mul(gu: torch.Tensor, F_: int, out_dtype: torch.dtype, kind: str,
     if kind == "copy":
         return g.to(out_dtype)
     u = gu[:, F_:2 * F_].float()
-    a = F.gelu(g, approximate="tanh") if kind == "gelu_mul" else F.silu(g)
+    a = (F.gelu(g, approximate="tanh") if kind == "gelu_mul" else
+         F.relu(g) if kind == "relu_mul" else F.silu(g))
     return (a * u).to(out_dtype)
 
 
@@ -701,6 +702,14 @@ def side_gate(gate, ids, table, col0, out_dtype):
     return (F.gelu(gate.float(), approximate="tanh") * e).to(out_dtype)
 
 
+def gated_rmsnorm(src, gate, w, eps, groups, out_dtype):
+    """RMS norm of src * silu(gate) (fp32 [T, n] both) in ``groups`` equal parts, times w [n]."""
+    T, n = src.shape
+    v = (src.float() * F.silu(gate.float())).reshape(T, groups, n // groups)
+    v = v * torch.rsqrt(v.pow(2).mean(-1, keepdim=True) + eps)
+    return (v.reshape(T, n) * w.float()).to(out_dtype)
+
+
 def rmsnorm_cols(src, w, eps, out_dtype, gate=None):
     """Rows of the fp32 (column-sliced) matrix ``src`` divided by their RMS, times w (and times
     sigmoid(gate), an fp32 matrix of the same shape, when given)."""
@@ -986,18 +995,36 @@ def rotate_by_table(x, table, rot_dims):
     return torch.cat([u * c - v * s, v * c + u * s, x[..., rot_dims:]], -1)
 
 
-def rope_prepare(proj, bias, table, rot_dims, H, G, d, dv, kcache, vcache, slots, out_dtype, tied):
+def rotate_adjacent_by_table(x, table, rot_dims):
+    """x [T, heads, n]: dimension 2i < rot_dims of every head turns with 2i + 1."""
+    if not rot_dims:
+        return x
+    h = rot_dims // 2
+    c, s = table[:, None, :h], table[:, None, h:]
+    u, v = x[..., 0:rot_dims:2], x[..., 1:rot_dims:2]
+    y = torch.stack([u * c - v * s, v * c + u * s], -1).reshape(*x.shape[:-1], rot_dims)
+    return torch.cat([y, x[..., rot_dims:]], -1)
+
+
+def rope_prepare(proj, bias, table, rot_dims, H, G, d, dv, kcache, vcache, slots, out_dtype, tied,
+                 adjacent=False, own_kv=True):
     """proj fp32 [T, q | k (| v)] (+ bias [that width]): q and k heads rotated by ``table``;
     rotated k -> kcache rows; v, or with ``tied`` the unrotated k, -> vcache rows; returns q
-    [T, H*d]."""
+    [T, H*d]. Without ``own_kv`` there are queries only."""
     T = proj.shape[0]
+    turn = rotate_adjacent_by_table if adjacent else rotate_by_table
+    if not own_kv:
+        p = proj[:, :H * d].float()
+        if bias is not None:
+            p = p + bias.float()
+        return turn(p.reshape(T, H, d), table, rot_dims).reshape(T, H * d).to(out_dtype)
     n = (H + G) * d + (0 if tied else G * dv)
     p = proj[:, :n].float()
     if bias is not None:
         p = p + bias.float()
-    q = rotate_by_table(p[:, :H * d].reshape(T, H, d), table, rot_dims)
+    q = turn(p[:, :H * d].reshape(T, H, d), table, rot_dims)
     kraw = p[:, H * d:(H + G) * d]
-    k = rotate_by_table(kraw.reshape(T, G, d), table, rot_dims)
+    k = turn(kraw.reshape(T, G, d), table, rot_dims)
     v = kraw if tied else p[:, (H + G) * d:]
     ok = slots >= 0
     idx = slots[ok].long()
@@ -1035,3 +1062,87 @@ def retention(proj, table, rot_dims, decays, eps, state, slots, cu_seqlens, posi
             out[t] = o.reshape(H * dv) * F.silu(g[t])
         state[sl[s]] = S
     return out.to(out_dtype)
+
+
+# ----------------------------------------------------------------------------- sandwich-norm designs
+def unit_rms(x, eps):
+    return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps)
+
+
+def sandwich_add(x, y, w_post, eps, w_next, w_offset, out_dtype):
+    """In place on the fp32 stream: x += rms(y) * (w_post + w_offset); returns the RMS norm of the
+    new x times (w_next + w_offset), None without w_next. y fp32 [T, D]."""
+    x.add_(unit_rms(y.float(), eps) * (w_post.float() + w_offset))
+    if w_next is None:
+        return None
+    return (unit_rms(x, eps) * (w_next.float() + w_offset)).to(out_dtype)
+
+
+def mean_of_normed(left, right, wl, wr, eps):
+    """Half the sum of two fp32 matrices' RMS-normed rows, each times its weight."""
+    return 0.5 * (unit_rms(left.float(), eps) * wl.float() + unit_rms(right.float(), eps) * wr.float())
+
+
+def sigmoid_router(h, w_router, top):
+    """The ``top`` experts with the largest fp32 logits h @ w^T (lowest index on ties) and the
+    sigmoids of their logits: (weights fp32 [T, top], ids int32 [T, top])."""
+    z = h.float() @ w_router.float().t()
+    order = torch.sort(z, dim=-1, descending=True, stable=True)
+    return torch.sigmoid(order.values[:, :top]), order.indices[:, :top].to(torch.int32)
+
+
+def moe_weighed_inputs_f32(x, w_gu, w_down, topk_w, topk_ids, shared=None):
+    """Sum of every token's chosen gated-SiLU experts, each on the token's row times its weight,
+    fp32; ``shared`` = (ws_gu, ws_down) adds the always-on expert of the plain row."""
+    T, D = x.shape
+    out = torch.zeros(T, D, dtype=torch.float32)
+    for e in range(w_gu.shape[0]):
+        rows, slot = (topk_ids == e).nonzero(as_tuple=True)
+        if rows.numel() == 0:
+            continue
+        xs = (x[rows].float() * topk_w[rows, slot][:, None]).to(x.dtype)
+        a = act_mul(linear(xs, w_gu[e], out_dtype=torch.float32), w_gu.shape[1] // 2, x.dtype, "silu_mul")
+        out.index_add_(0, rows, linear(a, w_down[e], out_dtype=torch.float32))
+    if shared is not None:
+        a = act_mul(linear(x, shared[0], out_dtype=torch.float32), shared[0].shape[0] // 2, x.dtype,
+                    "silu_mul")
+        out += linear(a, shared[1], out_dtype=torch.float32)
+    return out
+
+
+def ssd(xbc, dt, conv_w, conv_b, dt_bias, rate, skip, state, conv, slots, cu_seqlens, positions,
+        H, N, P, G):
+    """State-space recurrence over per-sequence slots. xbc fp32 [T, H*P + 2*G*N] = [x | B | C]
+    before the convolution, dt fp32 [T, H]. Every channel is filtered by its ``taps`` latest
+    inputs (conv_w [channels, taps], the last column is the current token's; zeros before
+    position 0), plus conv_b, then SiLU. Per head h of group g: s = softplus(dt + dt_bias),
+    S = exp(-rate_h s) S + s B_g x^T, y = S^T C_g + skip_h x. state fp32 [slots, H, N, P];
+    conv fp32 [slots, taps, channels], row p mod taps = the input at position p. Returns y
+    [T, H*P] fp32; rows of sequences without a slot come out zero."""
+    T, taps = xbc.shape[0], conv_w.shape[1]
+    y = torch.zeros(T, H * P, dtype=torch.float32)
+    cu, sl = cu_seqlens.tolist(), slots.tolist()
+    rep = H // G
+    for s in range(len(cu) - 1):
+        t0, t1 = cu[s], cu[s + 1]
+        if t1 <= t0 or sl[s] < 0:
+            continue
+        p0, n = int(positions[t0]), t1 - t0
+        old = [conv[sl[s], (p0 - k) % taps] if p0 - k >= 0 else torch.zeros(xbc.shape[1])
+               for k in range(taps - 1, 0, -1)]
+        u = torch.cat([torch.stack(old) if old else xbc[:0].float(), xbc[t0:t1].float()], 0)
+        v = F.silu(sum(u[k:k + n] * conv_w[:, k].float() for k in range(taps)) + conv_b.float())
+        for t in range(max(0, n - taps), n):
+            conv[sl[s], (p0 + t) % taps] = xbc[t0 + t].float()
+        xv = v[:, :H * P].reshape(n, H, P)
+        B = v[:, H * P:H * P + G * N].reshape(n, G, N).repeat_interleave(rep, 1)
+        C = v[:, H * P + G * N:].reshape(n, G, N).repeat_interleave(rep, 1)
+        step = F.softplus(dt[t0:t1].float() + dt_bias.float(), threshold=1e9)
+        a = torch.exp(-rate.float() * step)
+        S = state[sl[s]].clone() if p0 else torch.zeros_like(state[sl[s]])
+        for t in range(n):
+            S = a[t][:, None, None] * S + (step[t][:, None] * B[t])[:, :, None] * xv[t][:, None, :]
+            o = torch.einsum("hnp,hn->hp", S, C[t]) + skip.float()[:, None] * xv[t]
+            y[t0 + t] = o.reshape(H * P)
+        state[sl[s]] = S
+    return y
