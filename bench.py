@@ -272,6 +272,45 @@ def run_design_bamudra(a):
                       "results": out}), flush=True)
 
 
+def run_design_lutovik(a):
+    """``--design lutovik``: prefill and decode throughput of the design at layer sizes of a
+    real model (random weights) beside a Mixtral of equal width, depth, heads, expert count,
+    expert width and experts per token, both through ``LLMEngine``. ``--design-vdim``: the value
+    width of the gated attention heads (their query / key width is 128). One JSON line."""
+    from dataclasses import replace
+    from distributed_llm_inferencing_amd.models.configs import LayerSpec, get_config, hybrid_config
+    D, Fw, V, Hh, G, hd = a.design_width, a.design_ff, 32000, a.design_width // 128, 8, 128
+    E, top, dv = 8, 2, a.design_vdim
+    moe = dict(ff_kind="moe", router="sigmoid", ff=Fw, experts=E, top=top, shared_ff=Fw // 7)
+    dense = dict(ff_kind="gated_relu", ff=top * Fw)
+    Hl = Hh * hd // dv                              # equal width of the concatenated heads
+    left = LayerSpec("rope_attention", heads=Hl, kv_heads=G * hd // dv, dim=hd, vdim=dv, scale=hd ** -0.5,
+                     window=1 << 30, rot_dims=hd, rot_base=500000.0, out_gate=True)
+    right = LayerSpec("ssd", heads=D // 64, dim=128, vdim=64, taps=4, groups=8, norm_parts=8)
+    sides = dict(heads=Hl, kv_heads=left.kv_heads, dim=hd, vdim=dv, left=left, right=right)
+    att = dict(heads=Hh, kv_heads=G, dim=hd, vdim=hd, scale=hd ** -0.5, window=1 << 30, rot_dims=64,
+               rot_base=500000.0, rot_adjacent=True, rot_llama3=(8.0, 1.0, 4.0, 8192.0))
+    hyb = hybrid_config("lutovik-bench", D, V,
+                        (LayerSpec("side_by_side", **sides, **dense),
+                         LayerSpec("rope_attention", **att, **moe),
+                         LayerSpec("rope_attention", kv_from=1, **att, **moe),
+                         LayerSpec("side_by_side", **sides, **moe)),
+                        arch="lutovik", max_position=1 << 15, norm_eps=1e-6, embed_scale=8.0,
+                        norm_offset=1.0, sandwich=True)
+    mix = replace(get_config("mixtral-8x7b"), name="mixtral-bench", hidden_size=D, num_layers=4,
+                  num_heads=Hh, num_kv_heads=G, head_dim=hd, intermediate_size=Fw, vocab_size=V,
+                  num_experts=E, top_k_experts=top, max_position=1 << 15)
+    out = _design_sweep((hyb, mix), a, V)
+    print(json.dumps({"metric": "prefill and decode tokens/s, Lutovik design vs Mixtral of equal "
+                                "size (random weights)", "unit": "tokens/s", "n_gpus": 1,
+                      "dtype": "bf16", "data": "synthetic prompts, random-init weights",
+                      "config": {"width": D, "expert_ff": Fw, "dense_ff": top * Fw,
+                                 "shared_ff": Fw // 7, "layers": 4, "heads": Hh, "kv_heads": G,
+                                 "head_dim": hd, "gated_heads": [Hl, hd, dv],
+                                 "ssd_heads": [D // 64, 128, 64], "experts": E, "top": top},
+                      "results": out}), flush=True)
+
+
 def run_design(a):
     """``--design buborax``: prefill and decode throughput of the hybrid design at layer sizes
     of a real model (random weights), beside a Llama of equal width, depth (= layer runs),
@@ -496,15 +535,18 @@ def main():
                     help="N>1: pp = layer-sharded pipeline (dense, default), ep = expert "
                          "parallel (MoE), tp = tensor-parallel ablation, dp = independent "
                          "replicas")
-    ap.add_argument("--design", default=None, choices=["buborax", "pulunex", "risutar", "lapunex", "bamudra"],
+    ap.add_argument("--design", default=None, choices=["buborax", "pulunex", "risutar", "lapunex", "bamudra",
+                                                       "lutovik"],
                     help="instead of the headline workload: prefill / decode throughput of "
                          "this design at real layer sizes beside the closest model of equal "
                          "size (buborax and bamudra: Llama, pulunex, risutar and lapunex: "
                          "Mixtral)")
-    ap.add_argument("--design-models", default="buborax,llama,pulunex,mixtral,risutar,lapunex,bamudra",
+    ap.add_argument("--design-models", default="buborax,llama,pulunex,mixtral,risutar,lapunex,bamudra,lutovik",
                     help="which of the design and its comparison model to run")
     ap.add_argument("--design-width", type=int, default=4096)
     ap.add_argument("--design-ff", type=int, default=14336)
+    ap.add_argument("--design-vdim", type=int, default=128, choices=[128, 256],
+                    help="value width of the gated heads (--design lutovik)")
     ap.add_argument("--design-window", type=int, default=1024)
     ap.add_argument("--design-prefill", type=_pairs, default=_pairs("4x2048,32x256"),
                     help="prompts x tokens, comma separated")
@@ -519,6 +561,8 @@ def main():
             return run_design_lapunex(a)
         if a.design == "bamudra":
             return run_design_bamudra(a)
+        if a.design == "lutovik":
+            return run_design_lutovik(a)
         return run_design_pulunex(a) if a.design == "pulunex" else run_design(a)
 
     from distributed_llm_inferencing_amd import launch

@@ -317,7 +317,7 @@ __global__ void __launch_bounds__(NTH) ssd_chunk_kernel(SsdArgs a) {
       const float* kp = Ks + (jt * 16 + fr) * ldq + 4 * q;
       const float* qp = Qs + (it * 16 + fr) * ldq + 4 * q;
       f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll (D ? 4 : 1)
+#pragma unroll 4
       for (int x = 0; x < N; x += 16) {
         const f32x4 kf = *reinterpret_cast<const f32x4*>(kp + x);
         const f32x4 qf = *reinterpret_cast<const f32x4*>(qp + x);
@@ -343,7 +343,7 @@ __global__ void __launch_bounds__(NTH) ssd_chunk_kernel(SsdArgs a) {
     {
       const float* vp = St + (ct * 16 + fr) * ldq + 4 * q;
       const float* qp = Qs + fr * ldq + 4 * q;
-#pragma unroll (D ? 4 : 1)
+#pragma unroll 4
       for (int x = 0; x < N; x += 16) {
         const f32x4 sf = *reinterpret_cast<const f32x4*>(vp + x);
 #pragma unroll
@@ -462,7 +462,7 @@ struct StepArgs {
 // A workgroup per (head, sequence). Thread = (column quad cq of QP, row group rg of RG = 256 / QP);
 // its R = ceil(N / RG) state quads stream through registers, all in flight at once. Every head
 // of a group filters the group's B and C for itself; the group's first head stores their inputs.
-template <int R>
+template <int R, int TAPS>
 __global__ void __launch_bounds__(256, R >= 32 ? 2 : 4) ssd_step_kernel(StepArgs a, int qp_log2) {
   extern __shared__ __attribute__((aligned(16))) float sm[];
   const int H = a.H, N = a.N, P = a.P, G = a.G;
@@ -483,6 +483,30 @@ __global__ void __launch_bounds__(256, R >= 32 ? 2 : 4) ssd_step_kernel(StepArgs
     return;
   }
   const int p = a.positions[t];
+  const int rep = H / G, g = h / rep, ch = H * P + 2 * G * N, ne = P + 2 * N;
+  const int taps = TAPS ? TAPS : a.taps;
+  const float* row = a.u + (long)t * a.ldu;
+  float* ring = a.ring + (long)slot * taps * ch;
+  const auto channel = [&](int e) {        // of this head's x, then its group's B, then its C
+    return e < P ? h * P + e : e < P + N ? H * P + g * N + (e - P) : H * P + (G + g) * N + (e - P - N);
+  };
+  // the filter's inputs (two elements a thread at most sizes) are on their way before the state's
+  constexpr int E = TAPS ? 2 : 1, KT = TAPS ? TAPS : 1;
+  float in[E][KT], wt[E][KT], bias[E];
+#pragma unroll
+  for (int u = 0; u < E; ++u) {
+    const int e = tid + 256 * u;
+    if (TAPS == 0 || e >= ne) continue;
+    const int c = channel(e);
+    bias[u] = a.b[c];
+    in[u][0] = row[c];
+#pragma unroll
+    for (int k = 1; k < KT; ++k)
+      in[u][k] = k <= p ? ring[(long)((p - k) % KT) * ch + c] : 0.f;
+#pragma unroll
+    for (int k = 0; k < KT; ++k) wt[u][k] = a.w[(long)c * KT + KT - 1 - k];
+  }
+  const float zdt = row[ch + h] + a.dt_bias[h], rate = a.rate[h];
   float* sp = a.state + ((long)slot * H + h) * N * P + 4 * cq;
   f32x4 S[R];
 #pragma unroll
@@ -491,23 +515,29 @@ __global__ void __launch_bounds__(256, R >= 32 ? 2 : 4) ssd_step_kernel(StepArgs
     S[i] = f32x4{0.f, 0.f, 0.f, 0.f};
     if (p != 0 && col && r < N) S[i] = *reinterpret_cast<const f32x4*>(sp + (long)r * P);
   }
-  const int rep = H / G, g = h / rep, ch = H * P + 2 * G * N;
-  const float* row = a.u + (long)t * a.ldu;
-  float* ring = a.ring + (long)slot * a.taps * ch;
-  for (int e = tid; e < P + 2 * N; e += 256) {
-    const bool own = e < P;
-    const int c = own ? h * P + e : e < P + N ? H * P + g * N + (e - P)
-                                              : H * P + (G + g) * N + (e - P - N);
-    const float cur = row[c];
-    const float* w = a.w + (long)c * a.taps;
-    float acc = a.b[c] + w[a.taps - 1] * cur;
-    for (int k = 1; k < a.taps && k <= p; ++k)
-      acc += w[a.taps - 1 - k] * ring[(long)((p - k) % a.taps) * ch + c];
-    if (own || h == g * rep) ring[(long)(p % a.taps) * ch + c] = cur;
+#pragma unroll
+  for (int u = 0; u < E; ++u) {
+    const int e = tid + 256 * u;
+    if (TAPS == 0 || e >= ne) continue;
+    float acc = bias[u];
+#pragma unroll
+    for (int k = 0; k < KT; ++k) acc += wt[u][k] * in[u][k];
+    if (e < P || h == g * rep) ring[(long)(p % KT) * ch + channel(e)] = in[u][0];
     sm[e] = silu32(acc);
   }
-  const float st = softplus32(row[ch + h] + a.dt_bias[h]);
-  const float dec = expf(-a.rate[h] * st);
+#pragma unroll 1
+  for (int e = tid + (TAPS ? 256 * E : 0); e < ne; e += 256) {
+    const int c = channel(e);
+    const float cur = row[c];
+    const float* w = a.w + (long)c * taps;
+    float acc = a.b[c] + w[taps - 1] * cur;
+    for (int k = 1; k < taps && k <= p; ++k)
+      acc += w[taps - 1 - k] * ring[(long)((p - k) % taps) * ch + c];
+    if (e < P || h == g * rep) ring[(long)(p % taps) * ch + c] = cur;
+    sm[e] = silu32(acc);
+  }
+  const float st = softplus32(zdt);
+  const float dec = expf(-rate * st);
   __syncthreads();
   f32x4 x = {0.f, 0.f, 0.f, 0.f};
   if (col) x = *reinterpret_cast<const f32x4*>(xs + 4 * cq);
@@ -526,6 +556,7 @@ __global__ void __launch_bounds__(256, R >= 32 ? 2 : 4) ssd_step_kernel(StepArgs
   __syncthreads();
   if (rg == 0 && col) {
     o = a.skip[h] * x;
+#pragma unroll 4
     for (int k = 0; k < RG; ++k) o += *reinterpret_cast<const f32x4*>(ov + (k * QP + cq) * 4);
     *reinterpret_cast<f32x4*>(yp) = o;
   }
@@ -595,10 +626,15 @@ extern "C" int dli_ssd_step(const float* u, int ldu, const float* w, const float
   if (R > 32 || sh > 48 * 1024) return (int)hipErrorNotSupported;
   StepArgs a{u, ldu, w, b, taps, dt_bias, rate, skip, state, ring, slots, cu, positions, y, H, N, P, G};
   dim3 grid(H, num_seqs);
-  if (R <= 1) ssd_step_kernel<1><<<grid, 256, sh, st>>>(a, lg);
-  else if (R <= 4) ssd_step_kernel<4><<<grid, 256, sh, st>>>(a, lg);
-  else if (R <= 8) ssd_step_kernel<8><<<grid, 256, sh, st>>>(a, lg);
-  else if (R <= 16) ssd_step_kernel<16><<<grid, 256, sh, st>>>(a, lg);
-  else ssd_step_kernel<32><<<grid, 256, sh, st>>>(a, lg);
+#define STEP_LAUNCH(RR)                                                              \
+  do {                                                                               \
+    if (taps == 4) ssd_step_kernel<RR, 4><<<grid, 256, sh, st>>>(a, lg);             \
+    else ssd_step_kernel<RR, 0><<<grid, 256, sh, st>>>(a, lg);                       \
+  } while (0)
+  if (R <= 1) STEP_LAUNCH(1);
+  else if (R <= 4) STEP_LAUNCH(4);
+  else if (R <= 16) STEP_LAUNCH(16);
+  else STEP_LAUNCH(32);
+#undef STEP_LAUNCH
   DLI_RETURN_LAUNCH();
 }

@@ -364,6 +364,11 @@ def calm_random_mixers(cfg: ModelConfig, params: Dict[str, torch.Tensor]) -> Non
         k = f"layers.{i}.wo"
         if s.kind == "lightning" and k in params:
             params[k].mul_(0.1)
+        # averaging many keys leaves nearly the same vector for every token, which a norm behind
+        # the mixer would raise to full size: its weight starts small
+        k = f"layers.{i}.norm1b"
+        if cfg.sandwich and k in params:
+            params[k].fill_(0.1 - cfg.norm_offset)
 
 
 def slice_experts(name: str, t: torch.Tensor, expert_range: Optional[tuple]) -> torch.Tensor:

@@ -107,7 +107,8 @@ _SIGS = {
     "dli_scalar_recurrence": [P, I, I, P, P, F, P, F, P, P, P, P, P, P, I, F, I, I, I, I, I,
                               I, P, I, P],
     # rotated designs (rotary.hip, retention.hip, swa_attention.hip)
-    "dli_swa_attention": [P, I, P, L, P, L, P, I, P, P, P, I, I, I, I, I, I, I, I, I, F, P, P],
+    "dli_swa_attention": [P, I, P, L, P, L, P, I, P, P, P, I, I, I, I, I, I, I, I, I, I, F, P, I, P,
+                          P],
     "dli_swa_attention_workspace_bytes": [I, I, I, I, I, I, I],
     "dli_sandwich_add": [P, P, I, I, L, P, I, P, P, F, P, I, I, P, P, P, I, I, F, F, I, P],
     "dli_gated_rmsnorm": [P, P, I, P, I, P, I, I, I, F, I, P],

@@ -356,17 +356,19 @@ def window_attention(q, k_cache, v_cache, dq, dv, H, G, cu_seqlens, max_seqlen, 
     hg = int(bool(head_gate))
     if q.dtype == torch.bfloat16 and MFMA_ATTENTION:
         lib = N.require_native()
-        if (dq == dv and Gk == G and not chunk and slopes is None and talk is None and gate is None
+        if (Gk == G and not chunk and slopes is None and talk is None and not head_gate
                 and sink is None and out_scale == 1.0):
-            # plain grouped-query attention: the dedicated kernels (head sizes 64 and 128)
-            nb = lib.dli_swa_attention_workspace_bytes(S, int(max_seqlen), H, G, dq, int(window),
+            # grouped-query attention, plain or with an elementwise output gate: the dedicated
+            # kernels (a few pairs of key and value widths)
+            nb = lib.dli_swa_attention_workspace_bytes(S, int(max_seqlen), H, G, dv, int(window),
                                                        int(keep_first))
             ws = _gemm.workspace(q.device, nb) if nb else None
             rc = lib.dli_swa_attention(
                 _p(q), q.stride(0), _p(k_cache), k_cache.stride(0), _p(v_cache),
                 v_cache.stride(0), _p(out), out.stride(0), _p(cu_seqlens), _p(positions),
                 _p(block_tables), block_tables.stride(0), block_size, S, int(max_seqlen), H, G, dq,
-                int(window), int(keep_first), float(scale), _p(ws), _st())
+                dv, int(window), int(keep_first), float(scale), _p(gate),
+                gate.stride(0) if gate is not None else 0, _p(ws), _st())
             if rc == 0:
                 return out
             if rc != _NOT_SUPPORTED:
@@ -975,8 +977,8 @@ def ssd(xbcdt, conv_w, conv_b, dt_bias, rate, skip, state, conv, slots, cu_seqle
         if rc != _NOT_SUPPORTED:
             raise RuntimeError(f"dli_ssd_step failed with hipError {rc}")
     chunked = N % 16 == 0 and N <= 256 and P % 4 == 0
-    # the convolved rows: bf16 when serving on the chunk form, else fp32
-    xdt = dtype if chunked else torch.float32
+    # the convolved rows: bf16 when serving on the chunk form (16-byte rows), else fp32
+    xdt = dtype if chunked and P % 8 == 0 else torch.float32
     xc = torch.empty(T, ch, dtype=xdt, device=xbcdt.device)
     _call("dli_ssd_conv", _p(xbcdt), xbcdt.stride(0), _p(conv_w), _p(conv_b), taps, _p(conv),
           _p(slots), _p(cu_seqlens), _p(positions), _p(xc), S, int(max_seqlen), ch, _dt(xdt), _st())
